@@ -39,13 +39,26 @@
  *                            ones (two mixers side by side), then the dynamic-tanh norm tanh(alpha x) w + b
  *   lv_qk_prep_store         lv_rotary_store with the pairing of rotated entries as a choice and an optional division of
  *                            every query and key head by its root mean square
- *   lv_masked_attn(_mfma)    lv_window_pool_attn(_mfma) with kept first tokens, chunked visibility and a learned sink per head
+ *   lv_masked_attn(_mfma)    lv_window_pool_attn(_mfma) with kept first tokens, chunked visibility, a learned sink per head and
+ *                            capped scores
  *   lv_lightning_attn        linear attention with a constant decay per head: S <- d S + k v^T, o = S^T q, state in f32
  *   lv_glu_act               act(gate) * up
  *   lv_moe_route_scored      lv_moe_route with softmax scores and groups ranked by their best expert as choices
  *   lv_expert_act_scale      lv_relu2_scale with the activation as a choice
  *   lv_moe_grouped_act_ff    lv_moe_grouped_ff with the activation as a choice and experts that hand their input through
  *   lv_scaled_row_add        y[t] += (sum of a token's factors) * h[t]
+ *   lv_causal_conv           short causal convolution over columns of a projection, optional bias and silu, with the carried
+ *                            inputs of every sequence read and replaced in the same launch
+ *   lv_conv_qkv_store        the same for the queries, keys and values of an attention layer: queries times a factor of their
+ *                            position, keys and values into the paged cache
+ *   lv_token_shift           mixes of every token's input with its predecessor's
+ *   lv_gated_scan            S <- decay S + write k v^T, o = S^T q with the state in f32, decay and write from step sizes,
+ *                            from log gates under a running maximum, or one decay per row of the state with a bonus
+ *   lv_scaled_head_norm_gate lv_head_norm_gate with a weight per head and a division of every head by its own number
+ *   lv_grouped_gate_norm     o * silu(z), RMS norm in equal parts, weight
+ *   lv_residual_pair_norm    single f32 residual: adds the scaled sum of two RMS-normed and weighted sublayer outputs, RMS norm
+ *   lv_embed_norm            scaled token row + hashed pair row + position row, RMS norm, the first sublayer's RMS norm
+ *   lv_unary_act             activation without a gate
  *
  * A "ragged step" is a batch of B sequences; sequence b brings cu_q[b+1]-cu_q[b] new tokens that
  * follow ctx_lens[b] tokens already in the cache / state (a whole prompt, a portion of one, or one
@@ -67,7 +80,7 @@
 extern "C" {
 #endif
 
-#define LV_MIX_ABI_VERSION 7
+#define LV_MIX_ABI_VERSION 8
 #define LV_MIX_BF16 0
 #define LV_MIX_F32 1
 #define LV_MIX_MAX_STREAMS 8
@@ -78,6 +91,10 @@ extern "C" {
 #define LV_MIX_ACT_RELU2 0        /* relu(z)^2 */
 #define LV_MIX_ACT_GELU_ERF 1     /* z Phi(z), exact */
 #define LV_MIX_ACT_GELU_TANH 2    /* 0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3))) */
+#define LV_MIX_ACT_TANH 3
+#define LV_MIX_SCAN_STEP 0        /* lv_gated_scan: how a state decays and what it takes, see there */
+#define LV_MIX_SCAN_LOG_GATES 1
+#define LV_MIX_SCAN_ROW_DECAY 2
 #define LV_MIX_SCORE_SIGMOID 0
 #define LV_MIX_SCORE_SOFTMAX 1
 #define LV_MIX_GROUP_TOP2_SUM 0   /* a group of experts is ranked by the sum of its two highest selection scores */
@@ -281,16 +298,17 @@ int lv_qk_prep_store(const void* proj, int64_t ld, int off_q, int off_k, int off
 /* lv_window_pool_attn with more ways to say what a query at position i sees among the cached positions j <= i:
  *   chunk == 0: i - j < window or j < keep_first;   chunk > 0: floor(i / chunk) == floor(j / chunk) or j < keep_first
  * (kept first tokens and chunks do not combine with pooled blocks, P > 0). sinks f32 [H] (may be NULL): the denominator of
- * head h's softmax also holds exp(sinks[h]); has_sink without sinks: exp(0). */
+ * head h's softmax also holds exp(sinks[h]); has_sink without sinks: exp(0). softcap > 0: the score q.k * scale becomes
+ * softcap * tanh(score / softcap). */
 int lv_masked_attn(const void* q, const void* k_cache, const void* v_cache, const void* kp, const void* vp,
                    const void* gate, int64_t ld_gate, void* out, const int32_t* cu_q, const int32_t* ctx_lens,
                    const int32_t* tok_seq, const int32_t* block_tables, int bt_stride, int64_t T, int H, int G, int D,
-                   int Dv, int page, int window, int keep_first, int chunk, int P, float scale, int has_sink,
+                   int Dv, int page, int window, int keep_first, int chunk, int P, float scale, float softcap, int has_sink,
                    const void* sinks, int64_t k_ld, int64_t v_ld, int gate_kind, int dtype, void* stream);
 int lv_masked_attn_mfma(const void* q, const void* k_cache, const void* v_cache, const void* kp, const void* vp,
                         const void* gate, int64_t ld_gate, void* out, const int32_t* cu_q, const int32_t* ctx_lens,
                         const int32_t* block_tables, int bt_stride, int B, int max_new_tokens, int H, int G, int D,
-                        int Dv, int page, int window, int keep_first, int chunk, int P, float scale, int has_sink,
+                        int Dv, int page, int window, int keep_first, int chunk, int P, float scale, float softcap, int has_sink,
                         const void* sinks, int nsplit, void* workspace, int64_t T, int64_t k_ld, int64_t v_ld,
                         int gate_kind, void* stream);
 
@@ -325,6 +343,72 @@ int lv_moe_combine_through(const void* rows, const void* inv, const void* weight
 /* y act [T, W] += (factors[t, 0] + ... + factors[t, nf - 1]) * h[t]; factors f32 rows of stride ld_f. */
 int lv_scaled_row_add(void* y, const void* h, const void* factors, int64_t ld_f, int nf, int64_t T, int W, int dtype,
                       void* stream);
+
+/* in act [T, >= C] with row stride ld; w f32 [C, taps] (last column = current token), bias f32 [C] or NULL; state act
+ * [slots, taps-1, C], the last inputs of every sequence, taken as zeros for a sequence with no context, replaced.
+ * out act [T, C] = sum_j w[:, j] u_(t-taps+1+j) + bias, through silu when `silu` is not 0.
+ * max_new_tokens = the largest cu_q[b+1] - cu_q[b] of the step. */
+int lv_causal_conv(const void* in, int64_t ld, const void* w, const void* bias, void* state, const int32_t* cu_q,
+                   const int32_t* ctx_lens, const int32_t* slots, void* out, int B, int max_new_tokens, int C, int taps, int silu,
+                   int dtype, void* stream);
+
+/* The same (no bias, no silu) over columns [queries H*D | keys G*D | values G*Dv] of an attention layer. q_out act [T, H*D] =
+ * queries times 1 + temp_coef * ln(floor((pos + 1) / temp_every) + 1); keys and values into k_cache [pages, page, G, D] and
+ * v_cache [pages, page, G, Dv] at the token's slot. */
+int lv_conv_qkv_store(const void* in, int64_t ld, const void* w, void* state, void* q_out, void* k_cache, void* v_cache,
+                      const int32_t* cu_q, const int32_t* ctx_lens, const int32_t* slots, const int32_t* block_tables,
+                      int bt_stride, int B, int max_new_tokens, int H, int G, int D, int Dv, int taps, float temp_coef,
+                      int temp_every, int page, int dtype, void* stream);
+
+/* h act [T, W] contiguous, mu f32 [M, W], state act [slots, W] (each sequence's last row, zeros without context, replaced).
+ * out act [M, T, W] = h + (h' - h) * mu[m], h' = the previous token's row. */
+int lv_token_shift(const void* h, const void* mu, void* state, void* out, const int32_t* cu_q, const int32_t* ctx_lens,
+                   const int32_t* slots, const int32_t* tok_seq, int64_t T, int W, int M, int dtype, void* stream);
+
+/* Per head h (query/key group g = h / (H/G)) over the new tokens of every sequence, S f32 [D, Dv] in state [slots, H, D, Dv],
+ * taken as zero for a sequence with no context, written back. q, k act rows of G*D (strides ldq, ldk), v act rows of H*Dv.
+ *   LV_MIX_SCAN_STEP       a = step inputs, act rows of H (stride lda); p0 = their bias [H], p1 = log rates [H], p2 = skip [H]:
+ *                          dt = softplus(a + p0); S <- exp(-exp(p1) dt) S + dt k v^T; o = S^T (q_scale q) + p2 v
+ *   LV_MIX_SCAN_LOG_GATES  a, a2 = input and forget gates, act rows of H (stride lda); p0, p1 = their biases [H]:
+ *                          i = cap tanh((a + p0)/cap), f = logsigmoid(cap tanh((a2 + p1)/cap)); m' = max(f + m, i), m starts at 0;
+ *                          S <- e^(f+m-m') S + e^(i-m') k v^T, n <- e^(f+m-m') n + e^(i-m') k; o = S^T (q_scale q),
+ *                          den f32 [T, H] = max(|n . (q_scale q)|, e^(-m')) + 1e-6 (the caller divides).
+ *                          norm_state f32 [slots, H, D]; max_state f32 [slots, H, ceil(Dv / 64)]
+ *   LV_MIX_SCAN_ROW_DECAY  a = act rows of H*D (stride lda), p0 f32 [H*D], p1 = bonus f32 [H*D], G == H:
+ *                          w = exp(-exp(a + p0)); o = (S + diag(p1) k v^T)^T q; then S <- diag(w) S + k v^T
+ * o f32 [T, H, Dv]. D up to 256. All of this in f32. */
+int lv_gated_scan(int kind, const void* q, int64_t ldq, const void* k, int64_t ldk, const void* v, int64_t ldv, const void* a,
+                  const void* a2, int64_t lda, const void* p0, const void* p1, const void* p2, float q_scale, float cap,
+                  void* state, void* norm_state, void* max_state, const int32_t* cu_q, const int32_t* ctx_lens,
+                  const int32_t* slots, void* o, void* den, int B, int H, int G, int D, int Dv, int dtype, void* stream);
+
+/* lv_head_norm_gate with o[t, h] divided by den[t, h] first (den f32 [T, H] or NULL) and the norm weight of head h at
+ * norm_w + h * w_ld (w_ld 0: one weight for all heads; Dv: each its own). */
+int lv_scaled_head_norm_gate(const void* o, const void* den, const void* gate, int64_t ld_gate, const void* norm_w, int w_ld,
+                             void* out, int64_t T, int H, int Dv, float eps, int gate_act, int dtype, void* stream);
+
+/* o f32 [T, N], z act rows of stride ldz: y = o * silu(z); out act [T, N] = y / sqrt(mean(part^2) + eps) * w, each of the
+ * `groups` equal consecutive parts of the row by its own root mean square. */
+int lv_grouped_gate_norm(const void* o, const void* z, int64_t ldz, const void* w, void* out, int64_t T, int N, int groups,
+                         float eps, int dtype, void* stream);
+
+/* x f32 [T, W] += pair_scale * (y1 / rms(y1) * post_w1 + y2 / rms(y2) * post_w2), rms(y) = sqrt(mean(y^2) + pair_eps), in place;
+ * out act [T, W] = x / sqrt(mean(x^2) + eps) * (w_offset + w) (out may be NULL: update only). */
+int lv_residual_pair_norm(void* x, const void* y1, const void* post_w1, const void* y2, const void* post_w2, float pair_scale,
+                          float pair_eps, const void* w, float w_offset, void* out, int64_t T, int W, float eps, int dtype,
+                          void* stream);
+
+/* ids int64 [T]; table act [vocab, W]. e = table[id] * scale + pair_table[j] + pos_table[position] (act [buckets+1, W] and
+ * [max_pos, W], either may be NULL); j = (previous id * mul_prev + id * mul_cur) mod buckets, or `buckets` for a sequence's
+ * first token; prev_state int32 [slots] carries each sequence's last id.
+ * x f32 [T, W] = e / sqrt(mean(e^2) + eps) * (w_offset + w_embed);  out act [T, W] = x / sqrt(mean(x^2) + eps) * (w_offset + w_next). */
+int lv_embed_norm(const void* ids, const void* table, int vocab, float scale, const void* pair_table, int buckets,
+                  int64_t mul_prev, int64_t mul_cur, void* prev_state, const void* pos_table, int max_pos, const void* w_embed,
+                  const void* w_next, float w_offset, float eps, const int32_t* cu_q, const int32_t* ctx_lens,
+                  const int32_t* slots, const int32_t* tok_seq, void* x, void* out, int64_t T, int W, int dtype, void* stream);
+
+/* out act [n] = act(in), act one of LV_MIX_ACT_*. */
+int lv_unary_act(const void* in, void* out, int64_t n, int act, int dtype, void* stream);
 
 #ifdef __cplusplus
 }

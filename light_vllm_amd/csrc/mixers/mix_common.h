@@ -55,6 +55,19 @@ __device__ __forceinline__ float sigmoidf_(float x) { return 1.0f / (1.0f + expf
 __device__ __forceinline__ float siluf_(float x) { return x / (1.0f + expf(-x)); }
 __device__ __forceinline__ float softplusf_(float x) { return x > 20.0f ? x : log1pf(expf(x)); }
 
+__device__ __forceinline__ float gelu_tanh_(float z) {
+  return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
+}
+__device__ __forceinline__ float gelu_erf_(float z) { return 0.5f * z * (1.0f + erff(z * 0.7071067811865476f)); }
+
+__device__ __forceinline__ float mix_act(float v, int act) {
+  if (act == LV_MIX_ACT_GELU_ERF) return gelu_erf_(v);
+  if (act == LV_MIX_ACT_GELU_TANH) return gelu_tanh_(v);
+  if (act == LV_MIX_ACT_TANH) return tanhf(v);
+  v = fmaxf(v, 0.0f);
+  return v * v;
+}
+
 int fail(int code, const char* fmt, ...);
 inline hipStream_t as_stream(void* s) { return reinterpret_cast<hipStream_t>(s); }
 int launched(const char* what);

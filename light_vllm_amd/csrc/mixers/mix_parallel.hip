@@ -18,18 +18,6 @@
 
 namespace lvmix {
 
-__device__ __forceinline__ float gelu_tanh_(float z) {
-  return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
-}
-__device__ __forceinline__ float gelu_erf_(float z) { return 0.5f * z * (1.0f + erff(z * 0.7071067811865476f)); }
-
-__device__ __forceinline__ float expert_act(float v, int act) {
-  if (act == LV_MIX_ACT_GELU_ERF) return gelu_erf_(v);
-  if (act == LV_MIX_ACT_GELU_TANH) return gelu_tanh_(v);
-  v = fmaxf(v, 0.0f);
-  return v * v;
-}
-
 // two sums over the workgroup's four waves at once
 __device__ __forceinline__ void block_sum2(float& a, float& b, float (*red)[4]) {
   a = wave_sum(a);
@@ -384,10 +372,10 @@ __global__ __launch_bounds__(256) void glu_act_kernel(const T* __restrict__ in, 
   const T* row = in + t * ld_in;
   if constexpr (VEC == 4) {
     const float4 g = ld4(row + f), u = ld4(row + F + f);
-    st4(out + idx, float4{expert_act(g.x, act) * u.x, expert_act(g.y, act) * u.y, expert_act(g.z, act) * u.z,
-                          expert_act(g.w, act) * u.w});
+    st4(out + idx, float4{mix_act(g.x, act) * u.x, mix_act(g.y, act) * u.y, mix_act(g.z, act) * u.z,
+                          mix_act(g.w, act) * u.w});
   } else {
-    stf(out + idx, expert_act(ldf(row + f), act) * ldf(row + F + f));
+    stf(out + idx, mix_act(ldf(row + f), act) * ldf(row + F + f));
   }
 }
 
@@ -401,7 +389,7 @@ __global__ __launch_bounds__(256) void expert_act_scale_kernel(const T* __restri
   const int64_t t = idx / EF;
   const int e = static_cast<int>((idx - t * EF) / F);
   const float w = dense[t * ld_dense + e];
-  stf(out + idx, w != 0.0f ? expert_act(ldf(up + idx), act) * w : 0.0f);
+  stf(out + idx, w != 0.0f ? mix_act(ldf(up + idx), act) * w : 0.0f);
 }
 
 template <typename T>

@@ -15,7 +15,7 @@
 //                             each lane owns one column of the state, the four waves own a quarter of the
 //                             rows each, partial dot products meet in LDS once per token. The decay is one
 //                             number per head, or one for each key channel of it (a row of the state).
-//   head_norm_gate_kernel     one wave per (token, head).
+//   head_norm_gate_kernel     one wave per (token, head); optionally the head is divided by a number of its own first.
 #include "mix_common.h"
 
 namespace lvmix {
@@ -467,7 +467,8 @@ template <typename T>
 __global__ __launch_bounds__(256) void head_norm_gate_kernel(const float* __restrict__ o, const T* __restrict__ gate,
                                                              int64_t ld_gate, const float* __restrict__ norm_w,
                                                              T* __restrict__ out, int64_t items, int H, int Dv,
-                                                             float eps, int gate_act) {
+                                                             float eps, int gate_act, int w_ld,
+                                                             const float* __restrict__ den) {
   const int wave = threadIdx.x / kWave, lane = threadIdx.x % kWave;
   const int64_t item = static_cast<int64_t>(blockIdx.x) * (blockDim.x / kWave) + wave;   // (token, head)
   if (item >= items) return;
@@ -476,8 +477,10 @@ __global__ __launch_bounds__(256) void head_norm_gate_kernel(const float* __rest
   const float* row = o + item * Dv;
   float ss = 0.0f;
   for (int e = lane; e < Dv; e += kWave) ss += row[e] * row[e];
-  ss = wave_sum(ss);
-  const float inv = 1.0f / sqrtf(ss / static_cast<float>(Dv) + eps);
+  const float f = den != nullptr ? 1.0f / den[item] : 1.0f;     // the head is divided by its own number before the norm
+  ss = wave_sum(ss) * f * f;
+  const float inv = f / sqrtf(ss / static_cast<float>(Dv) + eps);
+  norm_w += static_cast<int64_t>(h) * w_ld;
   for (int e = lane; e < Dv; e += kWave) {
     const float gv = ldf(gate + t * ld_gate + h * Dv + e);
     stf(out + item * Dv + e, row[e] * inv * norm_w[e] * (gate_act == LV_MIX_GATE_SILU ? siluf_(gv) : sigmoidf_(gv)));
@@ -489,7 +492,8 @@ __global__ __launch_bounds__(256) void head_norm_gate_kernel(const float* __rest
 template <typename T>
 __global__ __launch_bounds__(256) void wide_head_norm_gate_kernel(const float* __restrict__ o, const T* __restrict__ gate,
                                                                   int64_t ld_gate, const float* __restrict__ norm_w,
-                                                                  T* __restrict__ out, int H, int Dv, float eps, int gate_act) {
+                                                                  T* __restrict__ out, int H, int Dv, float eps, int gate_act, int w_ld,
+                                                                  const float* __restrict__ den) {
   __shared__ float red[4];
   const int64_t item = blockIdx.x;
   const int64_t t = item / H;
@@ -503,7 +507,9 @@ __global__ __launch_bounds__(256) void wide_head_norm_gate_kernel(const float* _
   ss = wave_sum(ss);
   if (threadIdx.x % kWave == 0) red[threadIdx.x / kWave] = ss;
   __syncthreads();
-  const float inv = 1.0f / sqrtf(((red[0] + red[1]) + (red[2] + red[3])) / static_cast<float>(Dv) + eps);
+  const float f = den != nullptr ? 1.0f / den[item] : 1.0f;
+  const float inv = f / sqrtf(((red[0] + red[1]) + (red[2] + red[3])) * f * f / static_cast<float>(Dv) + eps);
+  norm_w += static_cast<int64_t>(h) * w_ld;
   const T* grow = gate + t * ld_gate + static_cast<int64_t>(h) * Dv;
   auto act = [&](float g) { return gate_act == LV_MIX_GATE_SILU ? siluf_(g) : sigmoidf_(g); };
   for (int e = threadIdx.x * 4; e < Dv; e += blockDim.x * 4) {
@@ -651,7 +657,13 @@ int lv_gated_delta_rule(const void* qn, const void* kn, const void* v, const voi
 
 int lv_head_norm_gate(const void* o, const void* gate, int64_t ld_gate, const void* norm_w, void* out, int64_t T,
                       int H, int Dv, float eps, int gate_act, int dtype, void* stream) {
+  return lv_scaled_head_norm_gate(o, nullptr, gate, ld_gate, norm_w, 0, out, T, H, Dv, eps, gate_act, dtype, stream);
+}
+
+int lv_scaled_head_norm_gate(const void* o, const void* den, const void* gate, int64_t ld_gate, const void* norm_w, int w_ld,
+                             void* out, int64_t T, int H, int Dv, float eps, int gate_act, int dtype, void* stream) {
   if (T == 0) return 0;
+  if (w_ld != 0 && w_ld != Dv) return fail(-1, "lv_head_norm_gate: weights of %d for heads of %d", w_ld, Dv);
   if (!o || !gate || !norm_w || !out || T < 0 || H <= 0 || Dv <= 0 || ld_gate < static_cast<int64_t>(H) * Dv ||
       (gate_act != LV_MIX_GATE_SILU && gate_act != LV_MIX_GATE_SIGMOID))
     return fail(-1, "lv_head_norm_gate: bad arguments");
@@ -663,22 +675,22 @@ int lv_head_norm_gate(const void* o, const void* gate, int64_t ld_gate, const vo
     if (dtype == LV_MIX_BF16)
       wide_head_norm_gate_kernel<bf16_t><<<wgrid, wblock, 0, as_stream(stream)>>>(
           static_cast<const float*>(o), static_cast<const bf16_t*>(gate), ld_gate, static_cast<const float*>(norm_w),
-          static_cast<bf16_t*>(out), H, Dv, eps, gate_act);
+          static_cast<bf16_t*>(out), H, Dv, eps, gate_act, w_ld, static_cast<const float*>(den));
     else
       wide_head_norm_gate_kernel<float><<<wgrid, wblock, 0, as_stream(stream)>>>(
           static_cast<const float*>(o), static_cast<const float*>(gate), ld_gate, static_cast<const float*>(norm_w),
-          static_cast<float*>(out), H, Dv, eps, gate_act);
+          static_cast<float*>(out), H, Dv, eps, gate_act, w_ld, static_cast<const float*>(den));
     return launched("lv_head_norm_gate");
   }
   dim3 grid(static_cast<unsigned>((items + 3) / 4)), block(256);
   if (dtype == LV_MIX_BF16)
     head_norm_gate_kernel<bf16_t><<<grid, block, 0, as_stream(stream)>>>(
         static_cast<const float*>(o), static_cast<const bf16_t*>(gate), ld_gate, static_cast<const float*>(norm_w),
-        static_cast<bf16_t*>(out), items, H, Dv, eps, gate_act);
+        static_cast<bf16_t*>(out), items, H, Dv, eps, gate_act, w_ld, static_cast<const float*>(den));
   else if (dtype == LV_MIX_F32)
     head_norm_gate_kernel<float><<<grid, block, 0, as_stream(stream)>>>(
         static_cast<const float*>(o), static_cast<const float*>(gate), ld_gate, static_cast<const float*>(norm_w),
-        static_cast<float*>(out), items, H, Dv, eps, gate_act);
+        static_cast<float*>(out), items, H, Dv, eps, gate_act, w_ld, static_cast<const float*>(den));
   else
     return fail(-1, "lv_head_norm_gate: dtype %d", dtype);
   return launched("lv_head_norm_gate");

@@ -89,6 +89,7 @@ struct WindowAttnParams {
   int keep_first;       // positions below this are seen from everywhere (with their own keys and values)
   int chunk;            // > 0: a query sees its own chunk of that many positions (counted from 0) up to itself; no window
   const float* sinks;   // [H] or NULL: a learned score per query head in place of the sink's 0
+  float softcap;        // > 0: scores pass softcap * tanh(score / softcap)
 };
 
 // kMaxRep: query heads of one kv head served by one workgroup; kMaxDvi: value columns per lane (Dv <= 64 * kMaxDvi).
@@ -164,6 +165,7 @@ __global__ __launch_bounds__(256) void window_pool_attn_kernel(WindowAttnParams 
 #pragma unroll
     for (int h = 0; h < kMaxRep; ++h) {
       if (h < rep) {
+        if (p.softcap > 0.0f) s[h] = p.softcap * tanhf(s[h] / p.softcap);
         const float cm = wave_max(valid ? s[h] : -INFINITY);
         const float nm = fmaxf(m[h], cm);
         const float corr = expf(m[h] - nm);
@@ -294,17 +296,18 @@ int lv_window_pool_attn(const void* q, const void* k_cache, const void* v_cache,
                         int Dv, int page, int window, int P, float scale, int has_sink, int64_t k_ld, int64_t v_ld,
                         int gate_kind, int dtype, void* stream) {
   return lv_masked_attn(q, k_cache, v_cache, kp, vp, gate, ld_gate, out, cu_q, ctx_lens, tok_seq, block_tables, bt_stride, T, H,
-                        G, D, Dv, page, window, 0, 0, P, scale, has_sink, nullptr, k_ld, v_ld, gate_kind, dtype, stream);
+                        G, D, Dv, page, window, 0, 0, P, scale, 0.0f, has_sink, nullptr, k_ld, v_ld, gate_kind, dtype, stream);
 }
 
 int lv_masked_attn(const void* q, const void* k_cache, const void* v_cache, const void* kp, const void* vp,
                    const void* gate, int64_t ld_gate, void* out, const int32_t* cu_q, const int32_t* ctx_lens,
                    const int32_t* tok_seq, const int32_t* block_tables, int bt_stride, int64_t T, int H, int G, int D,
-                   int Dv, int page, int window, int keep_first, int chunk, int P, float scale, int has_sink,
+                   int Dv, int page, int window, int keep_first, int chunk, int P, float scale, float softcap, int has_sink,
                    const void* sinks, int64_t k_ld, int64_t v_ld, int gate_kind, int dtype, void* stream) {
   if (T == 0) return 0;
   if (keep_first < 0 || chunk < 0 || (P > 0 && (keep_first > 0 || chunk > 0)))
     return fail(-1, "lv_masked_attn: kept first tokens and chunks do not combine with pooled blocks");
+  if (!(softcap >= 0.0f)) return fail(-1, "lv_masked_attn: softcap");
   if (sinks != nullptr) has_sink = 1;
   if (!q || !k_cache || !v_cache || !out || !cu_q || !ctx_lens || !tok_seq || !block_tables)
     return fail(-1, "lv_window_pool_attn: null pointer");
@@ -325,7 +328,7 @@ int lv_masked_attn(const void* q, const void* k_cache, const void* v_cache, cons
   WindowAttnParams p{q, k_cache, v_cache, kp, vp, gate, ld_gate, gate_dv, out, cu_q, ctx_lens, tok_seq, block_tables,
                      bt_stride, H, G, D, Dv, page, window, P, P > 0 ? (page + P - 1) / P : 0, scale,
                      has_sink ? 1.0f : 0.0f, k_ld, v_ld, has_sink ? 0.0f : -1e30f, keep_first, chunk,
-                     static_cast<const float*>(sinks)};
+                     static_cast<const float*>(sinks), softcap};
   const size_t shm = sizeof(float) * (static_cast<size_t>(kMaxRep) * D + 4 * kMaxRep * kWave +
                                       4 * static_cast<size_t>(kMaxRep) * Dv + 4 * kMaxRep * 2);
   if (shm > 64 * 1024) return fail(-2, "lv_window_pool_attn: head sizes %d / %d need %zu bytes of LDS", D, Dv, shm);

@@ -38,6 +38,7 @@ struct WindowMfmaParams {
   int keep_first;      // positions below this are seen from everywhere; they take the place of the pooled tiles (P == 0)
   int chunk;           // > 0: a query sees its own chunk of that many positions (counted from 0) up to itself; no window
   const float* sinks;  // [H] or NULL: a learned score per query head in place of the sink's 0
+  float cap_in, cap;   // CAP form: scores pass cap * tanh(product * cap_in), cap_in = scale / cap
 };
 
 constexpr int kTileQ = 16;
@@ -61,12 +62,15 @@ __device__ __forceinline__ short bf16_bits(float x) {
   return __builtin_bit_cast(short, b);
 }
 
+// tanh through the exponential: the absolute error stays at a few 1e-7, which is what a score multiplied by the cap needs.
+__device__ __forceinline__ float fast_tanh(float x) { return 1.0f - 2.0f * __builtin_amdgcn_rcpf(1.0f + __expf(2.0f * x)); }
+
 // AHEAD: the next tile's V rows, key-row addresses and (once the current scores are done) K fragments are fetched while
 // the current tile is computed. That pays when a launch has few workgroups per compute unit (decoded tokens). A prompt's
 // many tiles hide latency by occupancy instead, and every register counts there: with the 32 registers of a V tile held
 // ahead the kernel fell from two waves a SIMD to one and ran 1.7x slower; K32 and DVB size the fragment arrays for the
 // head sizes at hand for the same reason.
-template <bool AHEAD, int K32, int DVB>
+template <bool AHEAD, int K32, int DVB, bool CAP>
 __global__ __launch_bounds__(256, (AHEAD || DVB > 8) ? 1 : 4) void window_pool_mfma_kernel(WindowMfmaParams p) {
   extern __shared__ uint16_t vs[];                      // V^T tile [Dv][kLdk]
   const int wave = threadIdx.x / kWave, lane = threadIdx.x % kWave;
@@ -258,7 +262,7 @@ __global__ __launch_bounds__(256, (AHEAD || DVB > 8) ? 1 : 4) void window_pool_m
           bool vis = ke < e_end;
           if (phase == 0) vis = vis && (P == 0 || ke * P + P - 1 <= pos - W);
           else vis = vis && ke <= pos && ((chunk > 0 ? ke >= cstart : pos - ke < W) || ke < keep);
-          s[kb][i] = vis ? acc[i] * p.scale : -INFINITY;
+          s[kb][i] = vis ? (CAP ? p.cap * fast_tanh(acc[i] * p.cap_in) : acc[i] * p.scale) : -INFINITY;
         }
       }
       if (AHEAD && tile + 1 < t_end) fetch_k();                            // in flight across the softmax, PV and the barriers
@@ -375,19 +379,20 @@ extern "C" int lv_window_pool_attn_mfma(const void* q, const void* k_cache, cons
                                         float scale, int has_sink, int nsplit, void* workspace, int64_t T, int64_t k_ld,
                                         int64_t v_ld, int gate_kind, void* stream) {
   return lv_masked_attn_mfma(q, k_cache, v_cache, kp, vp, gate, ld_gate, out, cu_q, ctx_lens, block_tables, bt_stride, B,
-                             max_new_tokens, H, G, D, Dv, page, window, 0, 0, P, scale, has_sink, nullptr, nsplit, workspace, T,
+                             max_new_tokens, H, G, D, Dv, page, window, 0, 0, P, scale, 0.0f, has_sink, nullptr, nsplit, workspace, T,
                              k_ld, v_ld, gate_kind, stream);
 }
 
 extern "C" int lv_masked_attn_mfma(const void* q, const void* k_cache, const void* v_cache, const void* kp, const void* vp,
                                    const void* gate, int64_t ld_gate, void* out, const int32_t* cu_q, const int32_t* ctx_lens,
                                    const int32_t* block_tables, int bt_stride, int B, int max_new_tokens, int H, int G, int D,
-                                   int Dv, int page, int window, int keep_first, int chunk, int P, float scale, int has_sink,
+                                   int Dv, int page, int window, int keep_first, int chunk, int P, float scale, float softcap, int has_sink,
                                    const void* sinks, int nsplit, void* workspace, int64_t T, int64_t k_ld, int64_t v_ld,
                                    int gate_kind, void* stream) {
   if (B == 0 || max_new_tokens <= 0) return 0;
   if (keep_first < 0 || chunk < 0 || (P > 0 && (keep_first > 0 || chunk > 0)))
     return fail(-1, "lv_masked_attn_mfma: kept first tokens and chunks do not combine with pooled blocks");
+  if (!(softcap >= 0.0f)) return fail(-1, "lv_masked_attn_mfma: softcap");
   if (sinks != nullptr) has_sink = 1;
   if (!q || !k_cache || !v_cache || !out || !cu_q || !ctx_lens || !block_tables)
     return fail(-1, "lv_window_pool_attn_mfma: null pointer");
@@ -414,20 +419,27 @@ extern "C" int lv_masked_attn_mfma(const void* q, const void* k_cache, const voi
                      static_cast<uint16_t*>(out), cu_q, ctx_lens, block_tables, bt_stride, H, G, D, Dv, page, window, P,
                      P > 0 ? (page + P - 1) / P : 0, ngroups, scale, has_sink ? 1.0f : 0.0f,
                      magic(page), magic(P > 0 ? P : 1), magic(Dv / 4), nsplit > 1 ? nsplit : 1, static_cast<float*>(workspace),
-                     k_ld, v_ld, m0, keep_first, chunk, static_cast<const float*>(sinks)};
+                     k_ld, v_ld, m0, keep_first, chunk, static_cast<const float*>(sinks), softcap > 0.0f ? scale / softcap : 0.0f,
+                     softcap};
   if (nsplit > 1 && (max_new_tokens > kTileQ || workspace == nullptr || T <= 0))
     return fail(-1, "lv_window_pool_attn_mfma: key splits need one query tile per sequence and a workspace");
   const size_t shm = static_cast<size_t>(Dv) * kLdk * sizeof(uint16_t);
   dim3 grid(nsplit > 1 ? nsplit : (max_new_tokens + kTileQ - 1) / kTileQ, G * ngroups, B), block(256);
   hipStream_t st = as_stream(stream);
   const bool small = D <= 128 && Dv <= 128;
-  if (max_new_tokens <= kTileQ) {
-    if (small) window_pool_mfma_kernel<true, 4, 8><<<grid, block, shm, st>>>(p);
-    else window_pool_mfma_kernel<true, kMaxK32, kMaxDvb><<<grid, block, shm, st>>>(p);
-  } else {
-    if (small) window_pool_mfma_kernel<false, 4, 8><<<grid, block, shm, st>>>(p);
-    else window_pool_mfma_kernel<false, kMaxK32, kMaxDvb><<<grid, block, shm, st>>>(p);
-  }
+#define LVMIX_ATT(AHEAD)                                                                                  \
+  do {                                                                                                    \
+    if (softcap > 0.0f) {                                                                                 \
+      if (small) window_pool_mfma_kernel<AHEAD, 4, 8, true><<<grid, block, shm, st>>>(p);                 \
+      else window_pool_mfma_kernel<AHEAD, kMaxK32, kMaxDvb, true><<<grid, block, shm, st>>>(p);           \
+    } else {                                                                                              \
+      if (small) window_pool_mfma_kernel<AHEAD, 4, 8, false><<<grid, block, shm, st>>>(p);                \
+      else window_pool_mfma_kernel<AHEAD, kMaxK32, kMaxDvb, false><<<grid, block, shm, st>>>(p);          \
+    }                                                                                                     \
+  } while (0)
+  if (max_new_tokens <= kTileQ) LVMIX_ATT(true);
+  else LVMIX_ATT(false);
+#undef LVMIX_ATT
   if (nsplit > 1) {
     const int64_t items = T * H;
     window_pool_merge_kernel<<<dim3(static_cast<unsigned>((items + 3) / 4)), block, 0, st>>>(

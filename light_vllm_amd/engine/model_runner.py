@@ -315,11 +315,11 @@ class ModelRunner:
 
     # ------------------------------------------------------------------ step inputs
     def _check_positions(self, last_position: int) -> None:
-        """Positions index the rotary table (max_position_embeddings rows). The fused kernel clamps
-        instead of faulting, so the range is enforced here, where the lengths are known."""
+        """Positions index the rotary table or a learned position table (max_position_embeddings rows). The fused kernels
+        clamp instead of faulting, so the range is enforced here, where the lengths are known."""
         limit = getattr(self, "max_position", None)     # None: a bare runner built for its step-input builders
         if limit is not None and last_position >= limit:
-            raise IndexError(f"position {last_position} is outside the rotary table of {limit} rows "
+            raise IndexError(f"position {last_position} is outside the position table of {limit} rows "
                              "(sequence longer than max_position_embeddings)")
 
     def _to_device(self, values, dtype) -> torch.Tensor:
@@ -437,6 +437,7 @@ class ModelRunner:
             ctx_lens.append(ctx)
             lens_q.append(n)
             slots.append(seq.state_slot)
+        self._check_positions(max(c + n for c, n in zip(ctx_lens, lens_q)) - 1)
         if rows is None:
             rows = [c - 1 for c in cu_q[1:]]
         tables = [list(seq.block_table) for seq in seqs]
@@ -522,6 +523,7 @@ class ModelRunner:
         tables = self.prepare_block_tables(seqs)
         for seq in seqs:
             assert len(seq.block_table) * self.block_size >= seq.num_computed_tokens + 1 and seq.state_slot >= 0
+        self._check_positions(max(seq.num_computed_tokens for seq in seqs))
         gv["ctx_lens"][:bucket].zero_()
         gv["slots"][:bucket].fill_(self.pad_slot)
         gv["block_tables"][:bucket].fill_(self.pad_page)

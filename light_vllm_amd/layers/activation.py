@@ -1,6 +1,7 @@
 """SwiGLU: silu(gate) * up over the two halves of the last dim (reference "native" backend,
 lightvllm/layers/activation.py:7-29), the clamped gated unit with a sigmoid of slope alpha, PolyNorm,
-a learned cubic of the row-normalised powers of its input, and the gated unit with a choice of activation."""
+a learned cubic of the row-normalised powers of its input, the gated unit with a choice of activation, and that
+activation alone."""
 import torch
 import torch.nn.functional as F
 from torch import nn
@@ -53,3 +54,15 @@ class GatedAct(nn.Module):
 
     def forward(self, x: torch.Tensor) -> torch.Tensor:
         return mix_ops.glu_act(x, self.act)
+
+
+class Act(nn.Module):
+    """The activation without a gate: "relu2", "gelu", "gelu_tanh" or "tanh"."""
+
+    def __init__(self, act: str = "relu2"):
+        super().__init__()
+        assert act in mix_ops.ACTS
+        self.act = act
+
+    def forward(self, x: torch.Tensor) -> torch.Tensor:
+        return mix_ops.unary_act(x, self.act)

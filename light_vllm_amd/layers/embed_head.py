@@ -4,6 +4,8 @@ Embedding: each rank holds vocab rows [r*V/tp, (r+1)*V/tp), looks up its own ids
 and the ranks' partial rows are summed by all-reduce (:82-114). LM head: only the last token of
 each prefill sequence is projected (:161-167); per-rank logits [B, V/tp] are gathered to rank 0 and
 concatenated along the vocab axis (:175-195); other ranks return None.
+
+PairPositionEmbedding: an embedding that also looks at the previous token and the position.
 """
 from __future__ import annotations
 
@@ -12,6 +14,7 @@ import torch.distributed as dist
 import torch.nn.functional as F
 from torch import nn
 
+from .. import mix_ops
 from ..utils.context import get_context
 from . import tp
 from .tp import tp_rank, tp_size
@@ -46,6 +49,40 @@ class VocabParallelEmbedding(nn.Module):
             y = y * mask.unsqueeze(-1)
             tp.all_reduce(y)
         return y
+
+
+class PairPositionEmbedding(VocabParallelEmbedding):
+    """table[token] * scale + pair_table[(previous token * mul_prev + token * mul_cur) mod buckets] + pos_table[position],
+    then an RMS norm with weight (offset + w): the f32 residual a model starts from. A sequence's first token takes the pair
+    table's last row. `pair` = (buckets, mul_prev, mul_cur) or None, `positions` = rows of the position table or 0. Every
+    sequence's last token is state in its slot. `forward(ids, next_norm)` also returns the residual normed for the first
+    sublayer, all in one launch (mix_ops.embed_norm)."""
+    uses_state_slots = True
+
+    def __init__(self, num_embeddings: int, embedding_dim: int, scale: float = 1.0, pair: tuple | None = None, positions: int = 0,
+                 eps: float = 1e-6, offset: float = 1.0):
+        super().__init__(num_embeddings, embedding_dim)
+        assert self.tp_size == 1, "the pair embedding is not sharded: run it with tensor_parallel_size 1"
+        self.scale, self.eps, self.offset = float(scale), float(eps), float(offset)
+        self.buckets, self.mul_prev, self.mul_cur = (int(x) for x in pair) if pair is not None else (0, 0, 0)
+        assert pair is None or (self.buckets > 0 and self.mul_prev >= 0 and self.mul_cur >= 0)
+        self.pair_weight = nn.Parameter(torch.empty(self.buckets + 1, embedding_dim)) if pair is not None else None
+        self.pos_weight = nn.Parameter(torch.empty(positions, embedding_dim)) if positions > 0 else None
+        self.norm_weight = nn.Parameter(torch.zeros(embedding_dim, dtype=torch.float32))
+        self.prev_token = torch.tensor([])       # int32 [slots]
+
+    # -- cache protocol of the model runner
+    def cache_bytes(self, block_size: int, act_bytes: int) -> tuple[int, int]:
+        return 0, 4
+
+    def bind_cache(self, num_blocks: int, block_size: int, num_slots: int, device, dtype) -> None:
+        self.prev_token = torch.zeros(num_slots, dtype=torch.int32, device=device)
+
+    def forward(self, ids: torch.Tensor, next_norm: nn.Module):
+        assert next_norm.offset == self.offset and next_norm.eps == self.eps
+        return mix_ops.embed_norm(ids, self.weight, self.scale, self.pair_weight, self.buckets, self.mul_prev, self.mul_cur,
+                                  self.prev_token, self.pos_weight, self.norm_weight, next_norm.weight, self.offset, self.eps,
+                                  get_context().ragged)
 
 
 class ParallelLMHead(VocabParallelEmbedding):

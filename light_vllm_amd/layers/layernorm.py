@@ -47,14 +47,19 @@ class RMSNorm(nn.Module):
 class OffsetRMSNorm(nn.Module):
     """x / sqrt(mean(x^2) + eps) * (offset + w) on an f32 residual, fused with the residual update that
     precedes it: `forward(x, y1, y2)` adds up to two sublayer outputs to x in place and returns the normed
-    row in the activation dtype (mix_ops.residual_add_norm, one launch). The weight is f32."""
+    row in the activation dtype (mix_ops.residual_add_norm, one launch). With post weights the two outputs (of two mixers side
+    by side) are each divided by their root mean square and weighted, and x receives `pair_scale` times their sum
+    (mix_ops.residual_pair_norm). The weight is f32."""
 
     def __init__(self, hidden_size: int, eps: float = 1e-6, offset: float = 1.0):
         super().__init__()
         self.hidden_size, self.eps, self.offset = hidden_size, eps, float(offset)
         self.weight = nn.Parameter(torch.zeros(hidden_size, dtype=torch.float32))
 
-    def forward(self, x: torch.Tensor, y1=None, y2=None, act_dtype=None) -> torch.Tensor:
+    def forward(self, x: torch.Tensor, y1=None, y2=None, act_dtype=None, post_w1=None, post_w2=None, pair_scale: float = 1.0,
+                pair_eps: float = 1e-6) -> torch.Tensor:
+        if post_w1 is not None:
+            return mix_ops.residual_pair_norm(x, y1, y2, post_w1, post_w2, pair_scale, pair_eps, self.weight, self.offset, self.eps)
         return mix_ops.residual_add_norm(x, y1, y2, self.weight, self.offset, self.eps, act_dtype)
 
 

@@ -4,7 +4,8 @@ square over the model width and weighted, and the layer takes `scale` times thei
     y = scale * ( left(h) / rms(left(h)) * w_left + right(h) / rms(right(h)) * w_right )
 
 The two mixers are built with `fused_input`: their input projections are ONE GEMM here (the left one's columns, then
-the right one's; biases of a mixer that has none are zero). `forward` returns the two raw outputs; the norms, the
+the right one's; biases of a mixer that has none are zero). A mixer that projects something else than h (a mix of it with
+the previous token's, say) has no columns here (`sizes` empty) and projects for itself. `forward` returns the two raw outputs; the norms, the
 weights, the scale and the sum belong to the residual update that follows (mix_ops.residual_dyt), which reads
 `left_out`, `right_out`, `scale` and `eps` from this module.
 """

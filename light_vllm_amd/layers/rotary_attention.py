@@ -9,6 +9,7 @@ query head and a sigmoid output gate, on the paged cache of ragged steps.
     score_h(i, j) = q_h(i) . k_g(j) * scale * temp_h,  g = h / (H / G), over the positions j <= i that i sees:
         all of them; those with i - j < window; those of i's own chunk, floor(i / chunk) == floor(j / chunk);
         in each case also the first keep_first positions
+    with `softcap` a score becomes softcap * tanh(score / softcap)
     softmax over the visible keys, with `sink` the exponential of a learned number per head in the denominator as well
     o_h = sum_j p_h(i, j) v_g(j) * sigmoid(W_g h)_h              (gate: one number per head, per channel, or none)
     y = W_o [o_h]_h + b_o                                        (bias optional)
@@ -21,6 +22,11 @@ Prompts, portions of prompts and single decoded tokens are one code path.
 A module built with `share=` runs with the parameters of another one and keeps a cache of its own: the same
 layer applied again at another depth of the model. A module built with `fused_input` has no input projection: the
 caller hands `forward` the columns of a wider projection that it computed for several mixers at once.
+
+With `conv_taps` every channel of q, k and v passes a short causal convolution over time directly after the projection (no
+rotation, no unit norm and no head temperature then), and a query at position p can be multiplied by 1 + coef *
+ln(floor((p + 1) / every) + 1) (`q_temp`): one launch for the convolution, the factor and the cache writes
+(mix_ops.conv_qkv_store). The last conv_taps - 1 projected rows of each sequence are state in its slot.
 """
 from __future__ import annotations
 
@@ -42,7 +48,8 @@ class GatedRotaryAttention(nn.Module):
                  rot_base: float = 10000.0, rot_scaling: dict | None = None, bias: bool = True, head_temp: bool = True,
                  gate: str | None = "head", share: "GatedRotaryAttention | None" = None, interleaved: bool = False,
                  window: int = NO_WINDOW, keep_first: int = 0, chunk: int = 0, sink: bool = False,
-                 unit_norm_eps: float | None = None, out_bias: bool = False, fused_input: bool = False):
+                 unit_norm_eps: float | None = None, out_bias: bool = False, fused_input: bool = False, conv_taps: int = 0,
+                 q_temp: tuple | None = None, softcap: float = 0.0):
         super().__init__()
         assert tp_size() == 1, "the gated rotary attention is not sharded: run it with tensor_parallel_size 1"
         assert heads % kv_heads == 0 and gate in ("head", "channel", None)
@@ -51,6 +58,14 @@ class GatedRotaryAttention(nn.Module):
         self.scale, self.rot_dims, self.rot_base, self.rot_scaling = float(scale), rot_dims, float(rot_base), rot_scaling
         self.gate, self.bias, self.interleaved = gate, bias, interleaved
         self.window, self.keep_first, self.chunk, self.unit_norm_eps = window, keep_first, chunk, unit_norm_eps
+        self.conv_taps, self.softcap = conv_taps, float(softcap)
+        self.temp_coef, self.temp_every = (float(q_temp[0]), int(q_temp[1])) if q_temp is not None else (0.0, 1)
+        assert self.temp_every >= 1 and self.softcap >= 0.0
+        if conv_taps:
+            assert rot_dims == 0 and unit_norm_eps is None and not head_temp, "convolved q and k are neither rotated nor normed"
+        else:
+            assert q_temp is None, "the position's factor on the queries belongs to the convolved form"
+        self.uses_state_slots = conv_taps > 1
         gate_size = {"head": heads, "channel": heads * vdim, None: 0}[gate]
         self.sizes = [heads * dim, kv_heads * dim, kv_heads * vdim] + ([gate_size] if gate_size else [])
         if share is None:
@@ -62,20 +77,29 @@ class GatedRotaryAttention(nn.Module):
             self.o_proj = RowParallelLinear(heads * vdim, width, bias=out_bias)
             self.temp = nn.Parameter(torch.ones(heads, dtype=torch.float32)) if head_temp else None
             self.sink = nn.Parameter(torch.zeros(heads, dtype=torch.float32)) if sink else None
+            # channels q | k | v, last column: the current token
+            self.conv_weight = nn.Parameter(torch.zeros(sum(self.sizes[:3]), conv_taps, dtype=torch.float32)) if conv_taps else None
         else:
             assert (share.sizes, share.H, share.G, share.D, share.Dv) == (self.sizes, heads, kv_heads, dim, vdim)
             self.in_proj, self.o_proj, self.temp, self.sink = share.in_proj, share.o_proj, share.temp, share.sink
+            assert share.conv_taps == conv_taps
+            self.conv_weight = share.conv_weight
         self.inv_freq = None                         # f32 [rot_dims/2], made with the cache
         self.k_cache = self.v_cache = torch.tensor([])
 
     # -- cache protocol of the model runner
     def cache_bytes(self, block_size: int, act_bytes: int) -> tuple[int, int]:
-        return block_size * self.G * (self.D + self.Dv) * act_bytes, 0
+        conv = max(self.conv_taps - 1, 0) * sum(self.sizes[:3]) * act_bytes
+        return block_size * self.G * (self.D + self.Dv) * act_bytes, conv
 
     def bind_cache(self, num_blocks: int, block_size: int, num_slots: int, device, dtype) -> None:
         kw = dict(dtype=dtype, device=device)
         self.k_cache = torch.zeros(num_blocks, block_size, self.G, self.D, **kw)
         self.v_cache = torch.zeros(num_blocks, block_size, self.G, self.Dv, **kw)
+        if self.conv_taps:      # one tap: an empty view that still has an address
+            rows = self.conv_taps - 1
+            self._conv_buf = torch.zeros(num_slots, max(rows, 1), sum(self.sizes[:3]), **kw)
+            self.conv_state = self._conv_buf[:, :rows]
         self.inv_freq = mix_ops.rotary_inv_freq(max(self.rot_dims, 2), self.rot_base, device, self.rot_scaling)
 
     def forward(self, h: torch.Tensor, proj: torch.Tensor | None = None, col0: int = 0) -> torch.Tensor:
@@ -86,12 +110,16 @@ class GatedRotaryAttention(nn.Module):
         a = col0 + self.sizes[0]
         b = a + self.sizes[1]
         c = b + self.sizes[2]
-        q = mix_ops.rotary_store(proj, col0, a, b, self.inv_freq, self.temp, self.k_cache, self.v_cache, step,
-                                 self.H, self.G, self.D, self.Dv, self.rot_dims, interleaved=self.interleaved,
-                                 unit_eps=self.unit_norm_eps)
+        if self.conv_taps:
+            q = mix_ops.conv_qkv_store(proj[:, col0:c], self.conv_weight, self.conv_state, self.k_cache, self.v_cache, step, self.H,
+                                       self.G, self.D, self.Dv, self.temp_coef, self.temp_every)
+        else:
+            q = mix_ops.rotary_store(proj, col0, a, b, self.inv_freq, self.temp, self.k_cache, self.v_cache, step,
+                                     self.H, self.G, self.D, self.Dv, self.rot_dims, interleaved=self.interleaved,
+                                     unit_eps=self.unit_norm_eps)
         gate = proj[:, c:c + self.sizes[3]] if self.gate is not None else None
         o = mix_ops.window_pool_attention(q, self.k_cache, self.v_cache, None, None, gate, step, self.H, self.G, self.D,
                                           self.Dv, self.window, 0, self.scale, has_sink=False,
                                           gate_per_head=self.gate == "head", keep_first=self.keep_first, chunk=self.chunk,
-                                          sinks=self.sink)
+                                          sinks=self.sink, softcap=self.softcap)
         return self.o_proj(o)

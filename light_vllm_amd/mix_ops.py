@@ -395,7 +395,7 @@ def pool_update(k_cache, v_cache, kp, vp, step, G, D, Dv, P):
 
 
 def window_pool_attention(q, k_cache, v_cache, kp, vp, gate, step, H, G, D, Dv, window, P, scale, has_sink=True,
-                          gate_per_head=False, keep_first=0, chunk=0, sinks=None):
+                          gate_per_head=False, keep_first=0, chunk=0, sinks=None, softcap=0.0):
     """Query at position i attends to cached positions j with 0 <= i - j < window and to the pooled
     entry of every block b with b*P + P - 1 <= i - window, one softmax over both, `has_sink` adding 1
     to its denominator; the result is multiplied by sigmoid(gate) when a gate is given (gate rows hold
@@ -403,7 +403,7 @@ def window_pool_attention(q, k_cache, v_cache, kp, vp, gate, step, H, G, D, Dv, 
     keep_first > 0: positions j < keep_first are seen from everywhere as well. chunk > 0: instead of a window, a
     query sees the positions of its own chunk, floor(i / chunk) == floor(j / chunk), j <= i (chunks count from
     position 0 of the sequence). sinks f32 [H]: the denominator of head h holds exp(sinks[h]) instead of 1.
-    Neither combines with pooled blocks.
+    Neither combines with pooled blocks. softcap > 0: a score s = q.k * scale becomes softcap * tanh(s / softcap).
     q [T, H*D] contiguous act; returns act [T, H*Dv]. k_cache and v_cache [pages, page, G, D|Dv] may be
     views of wider token rows (one cache row serving as key and, in part, as value). A window that no
     sequence reaches, no pool and no sink give plain causal softmax attention."""
@@ -440,7 +440,7 @@ def window_pool_attention(q, k_cache, v_cache, kp, vp, gate, step, H, G, D, Dv, 
                                                   _p(step.ctx_lens), _p(step.block_tables),
                                                   step.block_tables.stride(0), len(step.host_lens_q),
                                                   max(step.host_lens_q), H, G, D, Dv, page, window, keep_first, chunk, P, scale,
-                                                  int(has_sink), _p(sinks), nsplit, _p(ws), T, k_ld, v_ld,
+                                                  softcap, int(has_sink), _p(sinks), nsplit, _p(ws), T, k_ld, v_ld,
                                                   0 if gate_per_head else 1, _stream(q)),
                           "lv_masked_attn_mfma")
             return out
@@ -448,7 +448,7 @@ def window_pool_attention(q, k_cache, v_cache, kp, vp, gate, step, H, G, D, Dv, 
                                          gate.stride(0) if gate is not None else 0, _p(out), _p(step.cu_q),
                                          _p(step.ctx_lens), _p(step.tok_seq), _p(step.block_tables),
                                          step.block_tables.stride(0), T, H, G, D, Dv, page, window, keep_first, chunk, P, scale,
-                                         int(has_sink), _p(sinks), k_ld, v_ld, 0 if gate_per_head else 1, _DT[q.dtype],
+                                         softcap, int(has_sink), _p(sinks), k_ld, v_ld, 0 if gate_per_head else 1, _DT[q.dtype],
                                          _stream(q)),
                       "lv_masked_attn")
         return out
@@ -470,6 +470,8 @@ def window_pool_attention(q, k_cache, v_cache, kp, vp, gate, step, H, G, D, Dv, 
                 V = torch.cat([vp.view(-1, G, Dv)[prow].float(), V])
             qi = q[q0 + r].float().view(G, rep, D)
             s = torch.einsum("grd,ngd->grn", qi, K) * scale
+            if softcap > 0:
+                s = softcap * torch.tanh(s / softcap)
             m = s.max(-1, keepdim=True).values
             sk = sinks.view(G, rep, 1) if sinks is not None else torch.zeros(G, rep, 1)
             if has_sink:
@@ -722,13 +724,15 @@ def moe_grouped_ok(h, Fe) -> bool:
     return h.dtype == torch.bfloat16 and h.size(1) % 32 == 0 and Fe % 32 == 0
 
 
-ACTS = {"relu2": 0, "gelu": 1, "gelu_tanh": 2}
+ACTS = {"relu2": 0, "gelu": 1, "gelu_tanh": 2, "tanh": 3}
 
 
 def _act(x, act):
-    """x f32 -> relu(x)^2, exact gelu, or the tanh form of gelu."""
+    """x f32 -> relu(x)^2, exact gelu, the tanh form of gelu, or tanh."""
     if act == "relu2":
         return torch.relu(x).pow(2)
+    if act == "tanh":
+        return torch.tanh(x)
     return F.gelu(x, approximate="tanh" if act == "gelu_tanh" else "none")
 
 
@@ -1009,3 +1013,306 @@ def lightning_attention(proj, off_q, off_k, off_v, decay, state, step, H, D, Dv)
         state[slot] = S
         q0 += n
     return o
+
+
+# ------------------------------------------------------- short convolutions, shifted tokens, gated scans
+def _conv_rows(x, w, bias, state, step):
+    """CPU restatement: f32 convolution of x act [T, C] with the carried inputs in state [slots, taps-1, C], which are
+    replaced by the last ones of every sequence."""
+    C, taps = w.shape
+    y = torch.empty(x.size(0), C)
+    q0 = 0
+    for b, (n, ctx) in enumerate(zip(step.host_lens_q, step.host_ctx_lens)):
+        slot = step.host_slots[b]
+        hist = state[slot].float() if ctx > 0 else torch.zeros(taps - 1, C)
+        full = torch.cat([hist, x[q0:q0 + n].float()])
+        y[q0:q0 + n] = sum(full[i:i + n] * w[:, i] for i in range(taps))
+        if bias is not None:
+            y[q0:q0 + n] += bias
+        if taps > 1:
+            state[slot] = full[-(taps - 1):].to(state.dtype)
+        q0 += n
+    return y
+
+
+def causal_conv(x, w, bias, state, step, silu=False):
+    """x act [T, C] (row stride free), w f32 [C, taps] (last column: the current token), bias f32 [C] or None, state act
+    [slots, taps-1, C]: y_t = sum_j w[:, j] x_(t-taps+1+j) + bias, through silu on request; what a portion does not hold
+    itself comes from the state (zeros for a sequence with no context), which is replaced by the sequence's last inputs.
+    Returns act [T, C]."""
+    T, C = x.shape
+    taps = w.size(1)
+    _f32(w, bias)
+    assert w.shape == (C, taps) and state.shape[1:] == (taps - 1, C) and state.is_contiguous() and state.dtype == x.dtype
+    out = torch.empty(T, C, dtype=x.dtype, device=x.device)
+    if x.is_cuda:
+        assert x.stride(1) == 1
+        lib = _mixlib.load()
+        _mixlib.check(lib.lv_causal_conv(_p(x), x.stride(0), _p(w), _p(bias), _p(state), _p(step.cu_q), _p(step.ctx_lens),
+                                         _p(step.slots), _p(out), len(step.host_lens_q), max(step.host_lens_q), C, taps,
+                                         int(silu), _DT[x.dtype], _stream(x)), "lv_causal_conv")
+        return out
+    y = _conv_rows(x, w, bias, state, step)
+    out.copy_(F.silu(y) if silu else y)
+    return out
+
+
+def conv_qkv_store(x, w, state, k_cache, v_cache, step, H, G, D, Dv, temp_coef=0.0, temp_every=1):
+    """x act [T, H*D + G*D + G*Dv] (row stride free) = projected queries | keys | values: causal_conv over all of them (no bias,
+    no silu), then the queries times 1 + temp_coef * ln(floor((position + 1) / temp_every) + 1), keys and values to the token's
+    row of the paged caches [pages, page, G, D|Dv]. Returns the queries, act [T, H*D]."""
+    T, C = x.shape
+    taps, page = w.size(1), k_cache.size(1)
+    _f32(w)
+    assert C == H * D + G * (D + Dv) and w.shape == (C, taps) and int(temp_every) == temp_every and temp_every >= 1
+    assert state.shape[1:] == (taps - 1, C) and state.is_contiguous() and state.dtype == x.dtype
+    assert k_cache.is_contiguous() and v_cache.is_contiguous() and k_cache.dtype == x.dtype and v_cache.dtype == x.dtype
+    q_out = torch.empty(T, H * D, dtype=x.dtype, device=x.device)
+    if x.is_cuda:
+        assert x.stride(1) == 1
+        lib = _mixlib.load()
+        _mixlib.check(lib.lv_conv_qkv_store(_p(x), x.stride(0), _p(w), _p(state), _p(q_out), _p(k_cache), _p(v_cache), _p(step.cu_q),
+                                            _p(step.ctx_lens), _p(step.slots), _p(step.block_tables),
+                                            step.block_tables.stride(0), len(step.host_lens_q), max(step.host_lens_q), H, G, D,
+                                            Dv, taps, float(temp_coef), int(temp_every), page, _DT[x.dtype], _stream(x)),
+                      "lv_conv_qkv_store")
+        return q_out
+    y = _conv_rows(x, w, None, state, step)
+    pos = _positions(step, x.device)
+    temp = 1.0 + temp_coef * torch.log(torch.div(pos + 1, int(temp_every), rounding_mode="floor").float() + 1.0)
+    q_out.copy_(y[:, :H * D] * temp[:, None])
+    kc, vc = k_cache.view(-1, G * D), v_cache.view(-1, G * Dv)
+    q0 = 0
+    for b, (n, ctx) in enumerate(zip(step.host_lens_q, step.host_ctx_lens)):
+        bt = step.host_block_tables[b]
+        for r in range(n):
+            sl = _token_slot(bt, ctx + r, page)
+            kc[sl] = y[q0 + r, H * D:H * D + G * D].to(kc.dtype)
+            vc[sl] = y[q0 + r, H * D + G * D:].to(vc.dtype)
+        q0 += n
+    return q_out
+
+
+def token_shift(h, mu, state, step):
+    """h act [T, W], mu f32 [M, W], state act [slots, W] (every sequence's last row, zeros without context; replaced):
+    act [M, T, W] = h + (h' - h) * mu[m] with h' the previous token's row of the same sequence."""
+    T, W = h.shape
+    M = mu.size(0)
+    _f32(mu)
+    assert mu.shape == (M, W) and state.shape[1] == W and state.dtype == h.dtype and state.is_contiguous()
+    out = torch.empty(M, T, W, dtype=h.dtype, device=h.device)
+    if h.is_cuda:
+        assert h.is_contiguous()
+        lib = _mixlib.load()
+        _mixlib.check(lib.lv_token_shift(_p(h), _p(mu), _p(state), _p(out), _p(step.cu_q), _p(step.ctx_lens), _p(step.slots),
+                                         _p(step.tok_seq), T, W, M, _DT[h.dtype], _stream(h)), "lv_token_shift")
+        return out
+    prev = torch.zeros_like(h)
+    q0 = 0
+    for b, (n, ctx) in enumerate(zip(step.host_lens_q, step.host_ctx_lens)):
+        slot = step.host_slots[b]
+        if ctx > 0:
+            prev[q0] = state[slot]
+        prev[q0 + 1:q0 + n] = h[q0:q0 + n - 1]
+        state[slot] = h[q0 + n - 1]
+        q0 += n
+    out.copy_(h.float() + (prev.float() - h.float()) * mu[:, None, :])
+    return out
+
+
+SCAN_STEP, SCAN_LOG_GATES, SCAN_ROW_DECAY = 0, 1, 2
+SCAN_COLUMNS = 64          # value columns of one workgroup of the scan (one copy of the running maximum each)
+
+
+def gated_scan(kind, q, k, v, a, p0, p1, step, state, H, G, D, Dv, a2=None, p2=None, q_scale=1.0, cap=1.0, norm_state=None,
+               max_state=None):
+    """State update S <- decay S + write k v^T and read-out o = S^T q per head over the new tokens of every sequence. q, k act
+    [T, G*D], v act [T, H*Dv] (row strides free, query/key group h // (H/G)); state f32 [slots, H, D, Dv], zero for a
+    sequence with no context, updated in place. `kind` says where decay and write come from:
+      SCAN_STEP       a act [T, H], p0 bias, p1 log rate, p2 skip (f32 [H]): dt = softplus(a + p0), decay = exp(-exp(p1) dt),
+                      write = dt, o += p2 v
+      SCAN_LOG_GATES  a, a2 act [T, H], p0, p1 their biases (f32 [H]): i = cap tanh((a + p0)/cap), f = logsigmoid(cap
+                      tanh((a2 + p1)/cap)), m' = max(f + m, i) with m from 0; decay = e^(f+m-m'), write = e^(i-m');
+                      n <- decay n + write k beside S. norm_state f32 [slots, H, D], max_state f32 [slots, H, ceil(Dv/64)]
+      SCAN_ROW_DECAY  a act [T, H*D], p0, p1 f32 [H*D]: w = exp(-exp(a + p0)) for each row of S; o = (S + diag(p1) k v^T)^T q
+                      before S <- diag(w) S + k v^T
+    q is multiplied by q_scale (not in SCAN_ROW_DECAY). Returns o f32 [T, H, Dv], and for SCAN_LOG_GATES also
+    max(|n . q|, e^(-m)) + 1e-6, f32 [T, H], which the caller divides by."""
+    T = q.size(0)
+    _f32(state, p0, p1, p2, norm_state, max_state)
+    assert state.shape[1:] == (H, D, Dv) and q.size(1) == G * D and k.size(1) == G * D and v.size(1) == H * Dv
+    assert a.size(1) == (H * D if kind == SCAN_ROW_DECAY else H) and a.dtype == q.dtype == k.dtype == v.dtype
+    o = torch.empty(T, H, Dv, dtype=torch.float32, device=q.device)
+    den = None
+    if kind == SCAN_LOG_GATES:
+        assert norm_state.shape[1:] == (H, D) and max_state.shape[1:] == (H, -(-Dv // SCAN_COLUMNS)) and a2.stride(0) == a.stride(0)
+        den = torch.empty(T, H, dtype=torch.float32, device=q.device)
+    if q.is_cuda:
+        assert all(x.stride(1) == 1 for x in (q, k, v, a))
+        lib = _mixlib.load()
+        _mixlib.check(lib.lv_gated_scan(kind, _p(q), q.stride(0), _p(k), k.stride(0), _p(v), v.stride(0), _p(a), _p(a2), a.stride(0),
+                                        _p(p0), _p(p1), _p(p2), float(q_scale), float(cap), _p(state), _p(norm_state),
+                                        _p(max_state), _p(step.cu_q), _p(step.ctx_lens), _p(step.slots), _p(o), _p(den),
+                                        len(step.host_lens_q), H, G, D, Dv, _DT[q.dtype], _stream(q)), "lv_gated_scan")
+        return (o, den) if den is not None else o
+    rep = H // G
+    Q = q.float().view(T, G, D).repeat_interleave(rep, 1)
+    K = k.float().view(T, G, D).repeat_interleave(rep, 1)
+    V = v.float().view(T, H, Dv)
+    af = a.float()
+    if kind != SCAN_ROW_DECAY:
+        Q = Q * q_scale
+    if kind == SCAN_STEP:
+        dt = F.softplus(af + p0)
+        dec, wr = torch.exp(-torch.exp(p1) * dt), dt
+    elif kind == SCAN_LOG_GATES:
+        li = cap * torch.tanh((af + p0) / cap)
+        lf = F.logsigmoid(cap * torch.tanh((a2.float() + p1) / cap))
+    else:
+        w = torch.exp(-torch.exp(af + p0.view(-1))).view(T, H, D)
+        u = p1.view(H, D)
+    q0 = 0
+    for b, (n, ctx) in enumerate(zip(step.host_lens_q, step.host_ctx_lens)):
+        slot = step.host_slots[b]
+        S = state[slot].clone() if ctx > 0 else torch.zeros(H, D, Dv)
+        if kind == SCAN_LOG_GATES:
+            ns = norm_state[slot].clone() if ctx > 0 else torch.zeros(H, D)
+            m = max_state[slot, :, 0].clone() if ctx > 0 else torch.zeros(H)
+        for t in range(q0, q0 + n):
+            kv = K[t][:, :, None] * V[t][:, None, :]
+            if kind == SCAN_ROW_DECAY:
+                o[t] = torch.einsum("hdv,hd->hv", S + u[:, :, None] * kv, Q[t])
+                S = w[t][:, :, None] * S + kv
+                continue
+            if kind == SCAN_STEP:
+                d_, w_ = dec[t], wr[t]
+            else:
+                nm = torch.maximum(lf[t] + m, li[t])
+                d_, w_, m = torch.exp(lf[t] + m - nm), torch.exp(li[t] - nm), nm
+                ns = d_[:, None] * ns + w_[:, None] * K[t]
+                den[t] = torch.maximum((ns * Q[t]).sum(-1).abs(), torch.exp(-m)) + 1e-6
+            S = d_[:, None, None] * S + w_[:, None, None] * kv
+            o[t] = torch.einsum("hdv,hd->hv", S, Q[t])
+            if kind == SCAN_STEP:
+                o[t] += p2[:, None] * V[t]
+        state[slot] = S
+        if kind == SCAN_LOG_GATES:
+            norm_state[slot] = ns
+            max_state[slot] = m[:, None]
+        q0 += n
+    return (o, den) if den is not None else o
+
+
+def scaled_head_norm_gate(o, gate, norm_w, eps, act_dtype, gate_act="silu", den=None):
+    """head_norm_gate with a norm weight for every head (norm_w f32 [H*Dv]) and, with den f32 [T, H], every head divided by
+    den[t, h] before its norm. o f32 [T, H, Dv] -> act [T, H*Dv]."""
+    assert gate_act in ("silu", "sigmoid")
+    T, H, Dv = o.shape
+    _f32(o, norm_w, den)
+    assert norm_w.numel() == H * Dv and (den is None or den.shape == (T, H))
+    out = torch.empty(T, H * Dv, dtype=act_dtype, device=o.device)
+    if o.is_cuda:
+        assert gate.stride(1) == 1 and gate.dtype == act_dtype and gate.size(1) == H * Dv
+        lib = _mixlib.load()
+        _mixlib.check(lib.lv_scaled_head_norm_gate(_p(o), _p(den), _p(gate), gate.stride(0), _p(norm_w), Dv, _p(out), T, H, Dv, eps,
+                                                   int(gate_act == "sigmoid"), _DT[act_dtype], _stream(o)),
+                      "lv_scaled_head_norm_gate")
+        return out
+    y = o / den[:, :, None] if den is not None else o
+    y = (y / torch.sqrt(y.pow(2).mean(-1, keepdim=True) + eps)).reshape(T, H * Dv) * norm_w
+    out.copy_(y * (F.silu(gate.float()) if gate_act == "silu" else torch.sigmoid(gate.float())))
+    return out
+
+
+def grouped_gate_norm(o, z, norm_w, groups, eps):
+    """o f32 [T, N], z act [T, N] (row stride free): y = o * silu(z), every one of the `groups` equal parts of the row divided
+    by its own sqrt(mean(part^2) + eps), times norm_w f32 [N]; returns act [T, N]."""
+    T, N = o.shape
+    _f32(o, norm_w)
+    assert z.shape == (T, N) and norm_w.numel() == N and N % groups == 0
+    out = torch.empty(T, N, dtype=z.dtype, device=o.device)
+    if o.is_cuda:
+        assert z.stride(1) == 1
+        lib = _mixlib.load()
+        _mixlib.check(lib.lv_grouped_gate_norm(_p(o), _p(z), z.stride(0), _p(norm_w), _p(out), T, N, groups, eps, _DT[z.dtype],
+                                               _stream(o)), "lv_grouped_gate_norm")
+        return out
+    y = (o * F.silu(z.float())).view(T, groups, N // groups)
+    y = y / torch.sqrt(y.pow(2).mean(-1, keepdim=True) + eps)
+    out.copy_(y.reshape(T, N) * norm_w)
+    return out
+
+
+def residual_pair_norm(x, y1, y2, post_w1, post_w2, pair_scale, pair_eps, w=None, w_offset=0.0, eps=1e-6):
+    """x [T, W] f32 += pair_scale * (y1 / rms(y1) * post_w1 + y2 / rms(y2) * post_w2) in place, rms(y) = sqrt(mean(y^2) +
+    pair_eps); returns x / sqrt(mean(x^2) + eps) * (w_offset + w) in the dtype of y1, or None when w is None."""
+    T, W = x.shape
+    _f32(x, post_w1, post_w2, w)
+    out = torch.empty(T, W, dtype=y1.dtype, device=x.device) if w is not None else None
+    if x.is_cuda:
+        for y in (y1, y2):
+            assert y.is_contiguous() and y.dtype == y1.dtype and y.shape == (T, W)
+        lib = _mixlib.load()
+        _mixlib.check(lib.lv_residual_pair_norm(_p(x), _p(y1), _p(post_w1), _p(y2), _p(post_w2), pair_scale, pair_eps, _p(w),
+                                                w_offset, _p(out), T, W, eps, _DT[y1.dtype], _stream(x)), "lv_residual_pair_norm")
+        return out
+    for y, pw in ((y1, post_w1), (y2, post_w2)):
+        yf = y.float()
+        x.add_(pair_scale * yf / torch.sqrt(yf.pow(2).mean(-1, keepdim=True) + pair_eps) * pw)
+    if w is None:
+        return None
+    out.copy_(x / torch.sqrt(x.pow(2).mean(-1, keepdim=True) + eps) * (w_offset + w))
+    return out
+
+
+def embed_norm(ids, table, scale, pair_table, buckets, mul_prev, mul_cur, prev_state, pos_table, w_embed, w_next, w_offset, eps,
+               step):
+    """ids int64 [T]: e = table[id] * scale + pair_table[j] + pos_table[position], with j = (previous id * mul_prev + id *
+    mul_cur) mod buckets, or `buckets` for a sequence's first token (pair_table [buckets + 1, W] and pos_table may be None;
+    prev_state int32 [slots] carries every sequence's last id). Returns x f32 [T, W] = rms_norm(e) * (w_offset + w_embed)
+    and rms_norm(x) * (w_offset + w_next) in the tables' dtype, all sums and norms in f32."""
+    T, W = ids.numel(), table.size(1)
+    _f32(w_embed, w_next)
+    assert pair_table is None or (pair_table.shape == (buckets + 1, W) and pair_table.dtype == table.dtype)
+    assert pos_table is None or (pos_table.size(1) == W and pos_table.dtype == table.dtype)
+    x = torch.empty(T, W, dtype=torch.float32, device=table.device)
+    out = torch.empty(T, W, dtype=table.dtype, device=table.device)
+    if table.is_cuda:
+        assert ids.dtype == torch.int64 and ids.is_contiguous() and table.is_contiguous()
+        assert prev_state is None or prev_state.dtype == torch.int32
+        lib = _mixlib.load()
+        _mixlib.check(lib.lv_embed_norm(_p(ids), _p(table), table.size(0), scale, _p(pair_table), buckets, mul_prev, mul_cur,
+                                        _p(prev_state), _p(pos_table), pos_table.size(0) if pos_table is not None else 0,
+                                        _p(w_embed), _p(w_next), w_offset, eps, _p(step.cu_q), _p(step.ctx_lens), _p(step.slots),
+                                        _p(step.tok_seq), _p(x), _p(out), T, W, _DT[table.dtype], _stream(table)), "lv_embed_norm")
+        return x, out
+    e = table[ids].float() * scale
+    if pair_table is not None:
+        rows = torch.empty(T, dtype=torch.long)
+        q0 = 0
+        for b, (n, ctx) in enumerate(zip(step.host_lens_q, step.host_ctx_lens)):
+            slot = step.host_slots[b]
+            prev = torch.cat([prev_state[slot:slot + 1].long(), ids[q0:q0 + n - 1]])
+            rows[q0:q0 + n] = (prev * mul_prev + ids[q0:q0 + n] * mul_cur) % buckets
+            if ctx == 0:
+                rows[q0] = buckets
+            prev_state[slot] = int(ids[q0 + n - 1])
+            q0 += n
+        e = e + pair_table[rows].float()
+    if pos_table is not None:
+        e = e + pos_table[_positions(step, table.device)].float()
+    x.copy_(e / torch.sqrt(e.pow(2).mean(-1, keepdim=True) + eps) * (w_offset + w_embed))
+    out.copy_(x / torch.sqrt(x.pow(2).mean(-1, keepdim=True) + eps) * (w_offset + w_next))
+    return x, out
+
+
+def unary_act(x, act="relu2"):
+    """act(x) element by element (relu2, gelu, gelu_tanh or tanh), computed in f32, in x's dtype."""
+    out = torch.empty_like(x)
+    if x.is_cuda:
+        assert x.is_contiguous()
+        lib = _mixlib.load()
+        _mixlib.check(lib.lv_unary_act(_p(x), _p(out), x.numel(), ACTS[act], _DT[x.dtype], _stream(x)), "lv_unary_act")
+        return out
+    out.copy_(_act(x.float(), act))
+    return out

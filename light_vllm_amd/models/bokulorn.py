@@ -25,7 +25,6 @@ from __future__ import annotations
 import json
 import os
 from dataclasses import dataclass, field
-from glob import glob
 from typing import Any, Optional
 
 import torch
@@ -36,21 +35,11 @@ from ..layers.embed_head import ParallelLMHead, VocabParallelEmbedding
 from ..layers.latent_attention import LatentAttention
 from ..layers.layernorm import OffsetRMSNorm
 from ..layers.moe import SparseMoE
+from ..utils.loader import tensor_shapes
 
 UNIT_NORM_EPS = 1e-6       # inside the root of the delta rule's unit norms
 NORM_WEIGHT_OFFSET = 1.0   # norm weights are offsets from one
 LATENT_TYPES = ("latent_attention", "latent_attention_2")
-
-
-def _tensor_shapes(path: str) -> dict:
-    """name -> shape of every tensor in the *.safetensors files of a directory (headers only)."""
-    from safetensors import safe_open
-    shapes = {}
-    for file in sorted(glob(os.path.join(path, "*.safetensors"))):
-        with safe_open(file, "pt", "cpu") as f:
-            for name in f.keys():
-                shapes[name] = tuple(f.get_slice(name).get_shape())
-    return shapes
 
 
 @dataclass
@@ -136,7 +125,7 @@ class BokulornConfig:
     @classmethod
     def from_pretrained(cls, path: str) -> "BokulornConfig":
         with open(os.path.join(path, "config.json")) as f:
-            return cls.from_dict(json.load(f), _tensor_shapes(path))
+            return cls.from_dict(json.load(f), tensor_shapes(path))
 
 
 def _make_mixer(config: BokulornConfig, spec: dict, share):

@@ -36,12 +36,18 @@ def _bisuzen():
     return BisuzenForCausalLM
 
 
+def _feditar():
+    from .feditar import FeditarForCausalLM
+    return FeditarForCausalLM
+
+
 MODELS = {
     "Qwen3ForCausalLM": _qwen3,
     "Kagalorn": _kagalorn,
     "Bokulorn": _bokulorn,
     "Givozen": _givozen,
     "Bisuzen": _bisuzen,
+    "Feditar": _feditar,
 }
 DEFAULT = "Qwen3ForCausalLM"
 

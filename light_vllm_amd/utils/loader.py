@@ -25,6 +25,17 @@ def checkpoint_tensors(path: str):
                 yield name, f.get_tensor(name)
 
 
+def tensor_shapes(path: str) -> dict:
+    """name -> shape of every tensor in the *.safetensors files of a directory (headers only)."""
+    from safetensors import safe_open
+    shapes = {}
+    for file in sorted(glob(os.path.join(path, "*.safetensors"))):
+        with safe_open(file, "pt", "cpu") as f:
+            for name in f.keys():
+                shapes[name] = tuple(f.get_slice(name).get_shape())
+    return shapes
+
+
 def load_model(model: nn.Module, path: str) -> None:
     from safetensors import safe_open
     if hasattr(model, "load_weights"):       # models with their own checkpoint naming place the tensors themselves
