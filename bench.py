@@ -1238,6 +1238,229 @@ def bisuzen_leg(sizes, batch, prompt_len, new_tokens, engine_only=False):
     print(json.dumps(out), flush=True)
 
 
+# --mixers-design feditar: the Feditar design (layers of matrix memory, of a state-space recurrence, and of attention with short
+# convolutions beside time mixing; squared-relu feed-forwards; an embedding that reads the previous token and the position)
+# beside Bisuzen, the closest existing model (two mixers side by side, a recurrent state per head in f32 behind one input
+# GEMM, the same paged attention kernel), at equal width, layer runs, state size per layer and active feed-forward parameters.
+FEDITAR_SIZES = {
+    "2k": dict(memory_heads=16, ssm_heads=32, ssm_vdim=64, ssm_state=128, ssm_groups=8, conv=4, mix_heads=32, mix_dim=64, decay_rank=64),
+    "4k": dict(memory_heads=32, ssm_heads=64, ssm_vdim=64, ssm_state=128, ssm_groups=8, conv=4, mix_heads=64, mix_dim=64, decay_rank=64),
+}
+
+
+def _feditar_config(z, fz):
+    from light_vllm_amd.models.feditar import FeditarConfig
+    D = z["dim"]
+    memory = {"heads": fz["memory_heads"], "dim": D, "vdim": D, "gate_cap": 15.0}
+    ssm = {"heads": fz["ssm_heads"], "vdim": fz["ssm_vdim"], "state": fz["ssm_state"], "groups": fz["ssm_groups"],
+           "norm_groups": fz["ssm_groups"], "conv": fz["conv"]}
+    pair = {"left": {"heads": z["heads"], "kv_heads": z["kv_heads"], "dim": D, "vdim": D, "scale": D ** -0.5, "conv": fz["conv"],
+                     "softcap": 30.0, "q_temp": {"coef": 0.1, "every": 512}},
+            "right": {"heads": fz["mix_heads"], "dim": fz["mix_dim"], "decay_rank": fz["decay_rank"]}}
+    kinds = [("parallel", pair), ("mlstm", memory), ("mamba2", ssm), ("mlstm", memory)]
+    layers = [{"type": kinds[i % 4][0], "mixer": kinds[i % 4][1], "mlp": {"kind": "dense", "ff": z["ff"]}}
+              for i in range(z["layers"])]
+    return FeditarConfig.from_dict({"vocab": z["vocab"], "width": z["width"], "norm": {"eps": 1e-6}, "max_positions": 8192,
+                                    "embedding": {"scale": z["width"] ** 0.5, "bigram": {"buckets": 65521, "mul_prev": 31, "mul_cur": 17}},
+                                    "layers": layers})
+
+
+def _graph_time(fn, calls=10, iters=5):
+    """Seconds per call on the device: `calls` of them replayed from one hipGraph, so that no launch waits for the host."""
+    with torch.inference_mode():
+        fn()
+        torch.cuda.synchronize()
+        graph = torch.cuda.CUDAGraph()
+        with torch.cuda.graph(graph):
+            for _ in range(calls):
+                fn()
+        return _event_time(graph.replay, iters, 2) / calls
+
+
+def _feditar_kernel_table(z, fz, sz, dev, batch, prompt_len):
+    """Each kernel of the design alone at one layer's shapes (prompt step and decode step), beside the kernel of Bisuzen (or, where
+    it has none, of another family) that does the like job."""
+    from light_vllm_amd import mix_ops
+    from light_vllm_amd.layers.rotary_attention import NO_WINDOW
+    from light_vllm_amd.utils.context import RaggedStep
+    bf = torch.bfloat16
+    W, H, G, D, Hs = z["width"], z["heads"], z["kv_heads"], z["dim"], sz["state_heads"]
+    page = 256
+    rows = []
+
+    def step_of(lens_q, ctx):
+        B = len(lens_q)
+        cu, tok = [0], []
+        for b, n_ in enumerate(lens_q):
+            cu.append(cu[-1] + n_)
+            tok += [b] * n_
+        per = -(-(max(ctx) + max(lens_q)) // page)
+        tables = [[b * per + j for j in range(per)] for b in range(B)]
+        i32 = dict(dtype=torch.int32, device=dev)
+        return RaggedStep(torch.tensor(cu, **i32), torch.tensor(ctx, **i32), torch.arange(B, **i32),
+                          torch.tensor(tok, **i32), torch.tensor(tables, **i32), lens_q, ctx, list(range(B)), tables), B * per
+
+    def add(name, phase, fn, nbytes=0, flops=0, like=None, matrix=False):
+        us = _graph_time(fn) * 1e6
+        rec = {"kernel": name, "phase": phase, "us": round(us, 1)}
+        if nbytes:
+            rec["of_hbm_roofline"] = round(nbytes / us / 1e3 / (HBM_BPS / 1e9), 3)
+        if flops:
+            rec["TFLOPs"] = round(flops / us / 1e6, 2)
+            if matrix:
+                rec["of_mfma_roofline"] = round(flops / us / 1e6 / (MFMA_FLOPS / 1e12), 4)
+        if like:
+            rec["like"] = like
+        rows.append(rec)
+
+    def rand(*shape, dtype=bf):
+        return torch.randn(*shape, device=dev, dtype=dtype)
+
+    Hm, Hx, Dx, N, Gx, taps = fz["memory_heads"], fz["ssm_heads"], fz["ssm_vdim"], fz["ssm_state"], fz["ssm_groups"], fz["conv"]
+    Hr, Dr = fz["mix_heads"], fz["mix_dim"]
+    inner = Hx * Dx
+    for phase, lens_q, ctx in (("prompt", [prompt_len] * batch, [0] * batch), ("decode", [1] * batch, [prompt_len] * batch)):
+        step, pages = step_of(lens_q, ctx)
+        T, B = sum(lens_q), len(lens_q)
+        decode = phase == "decode"
+        x = rand(T, W, dtype=torch.float32)
+        y1, y2 = rand(T, W), rand(T, W)
+        nw, alpha = torch.ones(W, device=dev), torch.full((1,), 0.5, device=dev)
+        # embedding and residual
+        table, pairs, posw = rand(z["vocab"], W), rand(65522, W), rand(8192, W)
+        ids = torch.randint(0, z["vocab"], (T,), device=dev)
+        prev = torch.zeros(B, dtype=torch.int32, device=dev)
+        add("embed_norm (three rows, two norms)", phase,
+            lambda: mix_ops.embed_norm(ids, table, 45.0, pairs, 65521, 31, 17, prev, posw, nw, nw, 1.0, 1e-6, step), nbytes=T * W * 12)
+        add("bisuzen embedding lookup, widening copy, norm", phase,
+            lambda: mix_ops.residual_dyt(torch.nn.functional.embedding(ids, table).float(), alpha=alpha, w=nw, b=nw, act_dtype=bf),
+            nbytes=T * W * 8, like="embed_norm")
+        add("residual_pair_norm", phase, lambda: mix_ops.residual_pair_norm(x, y1, y2, nw, nw, 0.5, 1e-6, nw, 1.0, 1e-6), nbytes=T * W * 14)
+        add("bisuzen residual_dyt (two normed mixer outputs)", phase,
+            lambda: mix_ops.residual_dyt(x, y1, y2, nw, nw, 0.5, 1e-6, alpha, nw, nw, bf), nbytes=T * W * 14, like="residual_pair_norm")
+        add("residual_add_norm", phase, lambda: mix_ops.residual_add_norm(x, y1, None, nw, 1.0, 1e-6, bf), nbytes=T * W * 12)
+        # attention inputs and attention
+        cols = H * D + 2 * G * D
+        proj = rand(T, cols)
+        kc = torch.zeros(pages, page, G, D, device=dev, dtype=bf)
+        vc = torch.zeros(pages, page, G, D, device=dev, dtype=bf)
+        cw = rand(cols, taps, dtype=torch.float32)
+        cstate = torch.zeros(B, taps - 1, cols, device=dev, dtype=bf)
+        conv_bytes = T * cols * 4 + cols * taps * 4 + B * (taps - 1) * cols * 4
+        add("conv_qkv_store", phase, lambda: mix_ops.conv_qkv_store(proj, cw, cstate, kc, vc, step, H, G, D, D, 0.1, 512), nbytes=conv_bytes)
+        inv_freq = mix_ops.rotary_inv_freq(sz["rot_dims"], 500000.0, dev)
+        add("bisuzen qk_prep_store", phase,
+            lambda: mix_ops.rotary_store(proj, 0, H * D, H * D + G * D, inv_freq, None, kc, vc, step, H, G, D, D, sz["rot_dims"],
+                                         interleaved=True), nbytes=T * cols * 4, like="conv_qkv_store")
+        q = mix_ops.conv_qkv_store(proj, cw, cstate, kc, vc, step, H, G, D, D, 0.1, 512)
+        keys = sum(i + 1 for n_, c0 in zip(lens_q, ctx) for i in range(c0, c0 + n_))
+        work = dict(nbytes=keys * G * D * 4) if decode else dict(flops=keys * H * D * 4, matrix=True)
+        add("attention with capped scores", phase,
+            lambda: mix_ops.window_pool_attention(q, kc, vc, None, None, None, step, H, G, D, D, NO_WINDOW, 0, D ** -0.5,
+                                                  has_sink=False, softcap=30.0), **work)
+        add("bisuzen attention, same keys", phase,
+            lambda: mix_ops.window_pool_attention(q, kc, vc, None, None, None, step, H, G, D, D, NO_WINDOW, 0, D ** -0.5,
+                                                  has_sink=False), like="attention with capped scores", **work)
+        # recurrences: the flops of one multiply-add into and one out of every entry of the state; bytes of the state when decoding
+        def scan_work(Hh, Dk, Dvv, in_bytes):
+            return dict(flops=T * Hh * Dk * Dvv * 4, nbytes=(B * Hh * Dk * Dvv * 8 + T * in_bytes) if decode else 0)
+        mproj = rand(T, 4 * Hm * D + 2 * Hm)
+        mq, mk, mv, mg = (mproj[:, j * Hm * D:(j + 1) * Hm * D] for j in range(4))
+        gi, gf = mproj[:, 4 * Hm * D:4 * Hm * D + Hm], mproj[:, 4 * Hm * D + Hm:]
+        ib, fb = torch.zeros(Hm, device=dev), torch.full((Hm,), 3.0, device=dev)
+        S1 = torch.zeros(B, Hm, D, D, device=dev)
+        n1, m1 = torch.zeros(B, Hm, D, device=dev), torch.zeros(B, Hm, -(-D // 64), device=dev)
+        add("gated_scan, log gates (matrix memory)", phase,
+            lambda: mix_ops.gated_scan(mix_ops.SCAN_LOG_GATES, mq, mk, mv, gi, ib, fb, step, S1, Hm, Hm, D, D, a2=gf, q_scale=D ** -0.5,
+                                       cap=15.0, norm_state=n1, max_state=m1), **scan_work(Hm, D, D, Hm * D * 10))
+        o, den = rand(T, Hm, D, dtype=torch.float32), torch.ones(T, Hm, device=dev)
+        gw = torch.ones(Hm * D, device=dev)
+        add("scaled_head_norm_gate (matrix memory)", phase, lambda: mix_ops.scaled_head_norm_gate(o, mg, gw, 1e-6, bf, "sigmoid", den=den),
+            nbytes=T * Hm * D * 8)
+        xproj = rand(T, 2 * inner + 2 * Gx * N + Hx)
+        C = inner + 2 * Gx * N
+        xw, xb = rand(C, taps, dtype=torch.float32), rand(C, dtype=torch.float32)
+        xstate = torch.zeros(B, taps - 1, C, device=dev, dtype=bf)
+        add("causal_conv (state space)", phase, lambda: mix_ops.causal_conv(xproj[:, inner:inner + C], xw, xb, xstate, step, silu=True),
+            nbytes=T * C * 4 + C * taps * 4 + B * (taps - 1) * C * 4)
+        dproj = rand(T, cols + 2 * Hs)
+        dA, db = torch.zeros(Hs, device=dev), torch.zeros(Hs, device=dev)
+        if Hs * D + 2 * G * D == cols:
+            dconv = torch.zeros(B, taps - 1, cols, device=dev, dtype=bf)
+            add("kagalorn delta_prep and conv_state_update", phase,
+                lambda: (mix_ops.delta_prep(dproj, cw, dconv, dA, db, step, G, Hs, D, D, taps, cols, dproj[:, cols + Hs:], 1e-6),
+                         mix_ops.conv_state_update(dproj, dconv, step, cols, taps)),
+                nbytes=T * cols * 6 + cols * taps * 4 + B * (taps - 1) * cols * 4, like="causal_conv, conv_qkv_store")
+        u = rand(T, C)
+        xs, xB, xC = torch.split(u, [inner, Gx * N, Gx * N], dim=1)
+        dt = xproj[:, inner + C:]
+        dtb, al, sk = torch.full((Hx,), -3.0, device=dev), torch.zeros(Hx, device=dev), torch.ones(Hx, device=dev)
+        S2 = torch.zeros(B, Hx, N, Dx, device=dev)
+        add("gated_scan, step sizes (state space)", phase,
+            lambda: mix_ops.gated_scan(mix_ops.SCAN_STEP, xC, xB, xs, dt, dtb, al, step, S2, Hx, Gx, N, Dx, p2=sk),
+            **scan_work(Hx, N, Dx, inner * 6 + Gx * N * 4))
+        xo = rand(T, inner, dtype=torch.float32)
+        xnw = torch.ones(inner, device=dev)
+        add("grouped_gate_norm (state space)", phase, lambda: mix_ops.grouped_gate_norm(xo, xproj[:, :inner], xnw, Gx, 1e-6), nbytes=T * inner * 8)
+        h = rand(T, W)
+        mu = torch.rand(5, W, device=dev)
+        sst = torch.zeros(B, W, device=dev, dtype=bf)
+        add("token_shift (five mixes)", phase, lambda: mix_ops.token_shift(h, mu, sst, step), nbytes=T * W * 12)
+        rkv = rand(4, T, Hr * Dr)
+        wr = rand(T, Hr * Dr)
+        w0, ub = torch.full((Hr * Dr,), -3.0, device=dev), torch.ones(Hr, Dr, device=dev)
+        S3 = torch.zeros(B, Hr, Dr, Dr, device=dev)
+        add("gated_scan, decay per row (time mixing)", phase,
+            lambda: mix_ops.gated_scan(mix_ops.SCAN_ROW_DECAY, rkv[0], rkv[1], rkv[2], wr, w0, ub, step, S3, Hr, Hr, Dr, Dr),
+            **scan_work(Hr, Dr, Dr, Hr * Dr * 12))
+        ro = rand(T, Hr, Dr, dtype=torch.float32)
+        rw = torch.ones(Hr * Dr, device=dev)
+        add("scaled_head_norm_gate (time mixing)", phase, lambda: mix_ops.scaled_head_norm_gate(ro, rkv[3], rw, 1e-6, bf, "silu"),
+            nbytes=T * Hr * Dr * 8)
+        lproj = rand(T, 4 * Hs * D)
+        decay = torch.full((Hs,), 0.99, device=dev)
+        S4 = torch.zeros(B, Hs, D, D, device=dev)
+        add("bisuzen lightning_attention", phase,
+            lambda: mix_ops.lightning_attention(lproj, 0, Hs * D, 2 * Hs * D, decay, S4, step, Hs, D, D), like="gated_scan",
+            **scan_work(Hs, D, D, Hs * D * 10))
+        # the same recurrence at the state shapes of the state-space and time-mixing layers
+        for Hh, Dk, Dvv in ((Hx, N, Dx), (Hr, Dr, Dr)):
+            lp, de, S5 = rand(T, 2 * Hh * Dk + Hh * Dvv), torch.full((Hh,), 0.99, device=dev), torch.zeros(B, Hh, Dk, Dvv, device=dev)
+            add(f"bisuzen lightning_attention at {Hh} heads of {Dk} x {Dvv}", phase,
+                lambda: mix_ops.lightning_attention(lp, 0, Hh * Dk, 2 * Hh * Dk, de, S5, step, Hh, Dk, Dvv), like="gated_scan",
+                **scan_work(Hh, Dk, Dvv, Hh * (2 * Dk + 3 * Dvv) * 2))
+        lo = rand(T, 1, Hs * D, dtype=torch.float32)
+        lw = torch.ones(Hs * D, device=dev)
+        add("bisuzen norm over all heads with gate", phase,
+            lambda: mix_ops.head_norm_gate(lo, lproj[:, 3 * Hs * D:], lw, 1e-6, bf, "sigmoid"), nbytes=T * Hs * D * 8,
+            like="scaled_head_norm_gate, grouped_gate_norm")
+        up = rand(T, z["ff"])
+        add("unary_act (squared relu)", phase, lambda: mix_ops.unary_act(up, "relu2"), nbytes=T * z["ff"] * 4)
+        zg = rand(T, 2 * z["ff"])
+        add("bisuzen glu_act", phase, lambda: mix_ops.glu_act(zg, "gelu_tanh"), nbytes=T * z["ff"] * 6, like="unary_act")
+    return rows
+
+
+def feditar_leg(sizes, batch, prompt_len, new_tokens, engine_only=False):
+    dev = torch.device("cuda:0")
+    torch.cuda.set_device(dev)
+    out = {"metric": "mixers: Feditar beside Bisuzen at equal size", "dtype": "bf16", "data": "synthetic, random weights",
+           "batch": batch, "prompt_len": prompt_len, "new_tokens": new_tokens, "sizes": []}
+    for name in sizes:
+        z, fz, sz = MIXER_SIZES[name], FEDITAR_SIZES[name], BISUZEN_SIZES[name]
+        rec = {"size": name, **z, **fz}
+        cache_tokens = batch * 256 * (-(-(prompt_len + new_tokens) // 256))
+        kw = dict(kvcache_block_size=256, max_cache_tokens=cache_tokens)
+        rec["feditar"] = _engine_rates(_feditar_config(z, fz), batch, prompt_len, new_tokens, **kw)
+        rec["feditar_graph"] = _engine_rates(_feditar_config(z, fz), batch, prompt_len, new_tokens, enforce_eager=False, **kw)
+        if not engine_only:
+            rec["bisuzen"] = _engine_rates(_bisuzen_config(z, sz), batch, prompt_len, new_tokens, **kw)
+            rec["bisuzen_graph"] = _engine_rates(_bisuzen_config(z, sz), batch, prompt_len, new_tokens, enforce_eager=False, **kw)
+            rec["kernels"] = _feditar_kernel_table(z, fz, sz, dev, batch, prompt_len)
+        out["sizes"].append(rec)
+    print(json.dumps(out), flush=True)
+
+
 def mixers_leg(sizes, batch, prompt_len, new_tokens):
     dev = torch.device("cuda:0")
     torch.cuda.set_device(dev)
@@ -1309,15 +1532,19 @@ def main():
                          "(proves launcher, rendezvous, graph and JSON path; not a measurement)")
     ap.add_argument("--mixers", default="", help="comma list of sizes (2k, 4k): instead of the default workload, "
                     "run the Kagalorn design beside Qwen3 at equal size and time its kernels one by one")
-    ap.add_argument("--mixers-design", default="kagalorn", choices=("kagalorn", "bokulorn", "givozen", "bisuzen"),
+    ap.add_argument("--mixers-design", default="kagalorn", choices=("kagalorn", "bokulorn", "givozen", "bisuzen", "feditar"),
                     help="with --mixers: kagalorn (beside Qwen3), bokulorn (beside Kagalorn, its closest relative) or "
-                         "givozen (beside Bokulorn, its closest relative) or bisuzen (beside Givozen, its closest relative)")
+                         "givozen (beside Bokulorn, its closest relative) or bisuzen (beside Givozen, its closest relative) or "
+                         "feditar (beside Bisuzen, its closest relative)")
     ap.add_argument("--mixers-engine-only", action="store_true",
-                    help="with --mixers-design bisuzen: only that design's engine runs (eager and from graphs), for a profiler")
+                    help="with --mixers-design bisuzen or feditar: only that design's engine runs (eager and from graphs), for a profiler")
     ap.add_argument("--mixers-batch", type=int, default=16)
     ap.add_argument("--mixers-prompt", type=int, default=1024)
     ap.add_argument("--mixers-new", type=int, default=17)
     args = ap.parse_args()
+    if args.mixers and args.mixers_design == "feditar":
+        return feditar_leg([x for x in args.mixers.split(",") if x], args.mixers_batch, args.mixers_prompt, args.mixers_new,
+                           args.mixers_engine_only)
     if args.mixers and args.mixers_design == "bisuzen":
         return bisuzen_leg([x for x in args.mixers.split(",") if x], args.mixers_batch, args.mixers_prompt, args.mixers_new,
                            args.mixers_engine_only)

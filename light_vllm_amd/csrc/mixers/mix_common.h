@@ -6,6 +6,8 @@
 #include <stdint.h>
 #include <stdio.h>
 
+#include <type_traits>
+
 #include "lv_mixers.h"
 
 namespace lvmix {
@@ -48,6 +50,19 @@ __device__ __forceinline__ float wave_sum(float x) {
 __device__ __forceinline__ float wave_max(float x) {
 #pragma unroll
   for (int o = 32; o > 0; o >>= 1) x = fmaxf(x, __shfl_xor(x, o, kWave));
+  return x;
+}
+
+// Sum over each aligned group of 16 lanes, left in all of them; lane permutations inside the vector ALU, no LDS traffic.
+__device__ __forceinline__ float row16_sum(float x) {
+  auto step = [&](auto ctrl) {
+    constexpr int c = decltype(ctrl)::value;
+    x += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, x), c, 0xf, 0xf, true));
+  };
+  step(std::integral_constant<int, 0xb1>{});      // lane ^ 1 within four
+  step(std::integral_constant<int, 0x4e>{});      // lane ^ 2 within four
+  step(std::integral_constant<int, 0x141>{});     // mirrored within eight
+  step(std::integral_constant<int, 0x140>{});     // mirrored within sixteen
   return x;
 }
 

@@ -5,7 +5,8 @@
 //                             silu, and carries the sequence's last inputs in the same launch. A second form hands the
 //                             result to attention: queries times a factor of their position, keys and values into the
 //                             paged caches. Long filters read their taps from memory instead.
-//   token_shift_kernel        every token's input mixed with its predecessor's by several weight vectors at once.
+//   token_shift_kernel        every token's input mixed with its predecessor's by several weight vectors at once; prompts take
+//                             tiles of tokens with the weights in registers.
 //   gated_scan_kernel         S <- decay S + write k v^T, o = S^T q per head over the new tokens of every sequence. What decays
 //                             and what is written are computed in f32 as the inputs are staged, from one of three rules:
 //                             step sizes of a state-space layer, log gates under a running maximum with a normaliser
@@ -204,6 +205,7 @@ static int conv_dispatch(const ConvParams& p, int B, int max_new, bool vec4, hip
 // ------------------------------------------------------------------------------------------------
 // out [M, T, W] = h + (h' - h) * mu[m], h' the previous token's row of the sequence. The workgroup of a sequence's first new
 // token is the only reader of the carried row and replaces it (each thread reads an element before it writes it).
+// Few tokens (decoded ones): a workgroup per token. Many, and M at most kShiftMax: below.
 template <typename T, int VEC>
 __global__ __launch_bounds__(256) void token_shift_kernel(const T* __restrict__ h, const float* __restrict__ mu, T* state,
                                                           T* __restrict__ out, const int32_t* __restrict__ cu_q,
@@ -239,6 +241,51 @@ __global__ __launch_bounds__(256) void token_shift_kernel(const T* __restrict__ 
   }
 }
 
+constexpr int kShiftMax = 5;
+constexpr int kShiftTile = 16;
+
+// Prompts: a thread keeps the weights of its four channels in registers and walks kShiftTile packed tokens, each row read once.
+template <typename T>
+__global__ __launch_bounds__(256) void token_shift_tile_kernel(const T* __restrict__ h, const float* __restrict__ mu, T* state,
+                                                               T* __restrict__ out, const int32_t* __restrict__ cu_q,
+                                                               const int32_t* __restrict__ ctx_lens,
+                                                               const int32_t* __restrict__ slots,
+                                                               const int32_t* __restrict__ tok_seq, int64_t Tn, int W, int M) {
+  const int i = (blockIdx.y * blockDim.x + threadIdx.x) * 4;
+  if (i >= W) return;
+  float f[kShiftMax][4];
+#pragma unroll
+  for (int m = 0; m < kShiftMax; ++m)
+    if (m < M) ldv<4>(mu + static_cast<int64_t>(m) * W + i, f[m]);
+  const int64_t t0 = static_cast<int64_t>(blockIdx.x) * kShiftTile, t1 = min(t0 + kShiftTile, Tn);
+  float prev[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+  if (t0 > 0) ldv<4>(h + (t0 - 1) * W + i, prev);
+  for (int64_t t = t0; t < t1; ++t) {
+    float cur[4];
+    ldv<4>(h + t * W + i, cur);
+    const int b = tok_seq[t];
+    if (t == cu_q[b]) {
+      T* srow = state + static_cast<int64_t>(slots[b]) * W + i;
+      if (ctx_lens[b] > 0) ldv<4>(srow, prev);
+      else prev[0] = prev[1] = prev[2] = prev[3] = 0.0f;
+      float last[4];
+      ldv<4>(h + static_cast<int64_t>(cu_q[b + 1] - 1) * W + i, last);
+      stv<4>(srow, last);
+    }
+#pragma unroll
+    for (int m = 0; m < kShiftMax; ++m) {
+      if (m < M) {
+        float y[4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) y[e] = cur[e] + (prev[e] - cur[e]) * f[m][e];
+        stv<4>(out + (static_cast<int64_t>(m) * Tn + t) * W + i, y);
+      }
+    }
+#pragma unroll
+    for (int e = 0; e < 4; ++e) prev[e] = cur[e];
+  }
+}
+
 // ------------------------------------------------------------------------------------------------
 enum ScanKind { kScanStep = LV_MIX_SCAN_STEP, kScanLogGates = LV_MIX_SCAN_LOG_GATES, kScanRowDecay = LV_MIX_SCAN_ROW_DECAY };
 
@@ -263,7 +310,8 @@ struct ScanShape {
   static constexpr int kDP = NW * DR;
   static constexpr int kChunk = kDP >= 256 ? 8 : 16;
   static constexpr int kSeg = kDP > kWave ? kDP / kWave : 1;         // partial sums of a token's bonus
-  static constexpr int kExtra = KIND == kScanStep ? 0 : kChunk * kDP;  // row decays, or shares of the normaliser's read-out
+  static constexpr int kRows16 = DR > 16 ? DR / 16 : 1;              // a wave's shares of the normaliser's read-out per token
+  static constexpr int kExtra = KIND == kScanStep ? 0 : (KIND == kScanRowDecay ? kChunk * kDP : kChunk * NW * kRows16);
   static constexpr size_t kLds = sizeof(float) * (2 * kChunk * kDP + kChunk * kWave + kChunk * NW * kWave + kExtra + 4 * kChunk +
                                                   kChunk * kSeg);
 };
@@ -272,10 +320,10 @@ template <typename T, int KIND, int DR, int NW>
 __global__ __launch_bounds__(NW * 64) void gated_scan_kernel(ScanParams p) {
   extern __shared__ __attribute__((aligned(16))) float sl[];
   using Shape = ScanShape<KIND, DR, NW>;
-  constexpr int DP = Shape::kDP, NT = NW * kWave, CH = Shape::kChunk, SEG = Shape::kSeg;
+  constexpr int DP = Shape::kDP, NT = NW * kWave, CH = Shape::kChunk, SEG = Shape::kSeg, R16 = Shape::kRows16;
   float* k_lds = sl;                               // [CH][DP]
   float* q_lds = k_lds + CH * DP;                  // [CH][DP]
-  float* x_lds = q_lds + CH * DP;                  // [CH][DP] row decays, or normaliser shares (absent for kScanStep)
+  float* x_lds = q_lds + CH * DP;                  // [CH][DP] row decays, or [CH][NW * R16] normaliser shares
   float* v_lds = x_lds + Shape::kExtra;            // [CH][64]
   float* part_o = v_lds + CH * kWave;              // [CH][NW][64]
   float* sc_lds = part_o + CH * NW * kWave;        // [CH][4]: decay, write, floor of the normaliser
@@ -404,10 +452,11 @@ __global__ __launch_bounds__(NW * 64) void gated_scan_kernel(ScanParams p) {
       if (KIND != kScanRowDecay) {
         const float2 dw = *reinterpret_cast<const float2*>(sc_lds + i * 4);
         dec = dw.x;
-        if (KIND == kScanLogGates && owner && lane < DR) {
-          const int at = i * DP + row0 + lane;
+        if (KIND == kScanLogGates && owner) {
+          const int at = i * DP + row0 + (lane < DR ? lane : 0);
           nstate = dec * nstate + dw.y * k_lds[at];
-          x_lds[at] = nstate * q_lds[at];
+          const float share = row16_sum(lane < DR ? nstate * q_lds[at] : 0.0f);
+          if (lane < DR && (lane & 15) == 0) x_lds[(i * NW + rp) * R16 + (lane >> 4)] = share;
         }
         vv *= dw.y;
       }
@@ -460,7 +509,7 @@ __global__ __launch_bounds__(NW * 64) void gated_scan_kernel(ScanParams p) {
       const int tok = threadIdx.x / PER, part = threadIdx.x % PER;
       float nq = 0.0f;
       if (tok < cn)
-        for (int d = part; d < DP; d += PER) nq += x_lds[tok * DP + d];
+        for (int d = part; d < NW * R16; d += PER) nq += x_lds[tok * NW * R16 + d];
 #pragma unroll
       for (int off = PER / 2; off > 0; off >>= 1) nq += __shfl_xor(nq, off, kWave);
       if (tok < cn && part == 0)
@@ -508,6 +557,45 @@ static void scan_kind(const ScanParams& p, int kind, int B, hipStream_t s) {
 }
 
 // ------------------------------------------------------------------------------------------------
+// Parts of at most 4 * 64 * kPartRegs entries, aligned: a wave per (token, part), the gated values in registers.
+constexpr int kPartRegs = 4;
+template <typename T>
+__global__ __launch_bounds__(256) void part_gate_norm_kernel(const float* __restrict__ o, const T* __restrict__ z, int64_t ldz,
+                                                             const float* __restrict__ w, T* __restrict__ out, int64_t items, int N,
+                                                             int groups, float eps) {
+  const int64_t item = static_cast<int64_t>(blockIdx.x) * (blockDim.x / kWave) + threadIdx.x / kWave;
+  if (item >= items) return;
+  const int64_t t = item / groups;
+  const int gs = N / groups, c0 = static_cast<int>(item - t * groups) * gs, i0 = 4 * (threadIdx.x % kWave);
+  float y[kPartRegs][4], ss = 0.0f;
+#pragma unroll
+  for (int x = 0; x < kPartRegs; ++x) {
+    const int i = i0 + x * 4 * kWave;
+    if (i < gs) {
+      float g[4];
+      ldv<4>(o + t * N + c0 + i, y[x]);
+      ldv<4>(z + t * ldz + c0 + i, g);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        y[x][e] *= siluf_(g[e]);
+        ss += y[x][e] * y[x][e];
+      }
+    }
+  }
+  const float inv = 1.0f / sqrtf(wave_sum(ss) / static_cast<float>(gs) + eps);
+#pragma unroll
+  for (int x = 0; x < kPartRegs; ++x) {
+    const int i = i0 + x * 4 * kWave;
+    if (i < gs) {
+      float ww[4];
+      ldv<4>(w + c0 + i, ww);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) y[x][e] *= inv * ww[e];
+      stv<4>(out + t * N + c0 + i, y[x]);
+    }
+  }
+}
+
 // One workgroup (64 or 256 threads) per (token, part of the row): y = o * silu(z), y / rms(part) * w.
 template <typename T, int VEC>
 __global__ __launch_bounds__(256) void grouped_gate_norm_kernel(const float* __restrict__ o, const T* __restrict__ z, int64_t ldz,
@@ -760,6 +848,21 @@ int lv_token_shift(const void* h, const void* mu, void* state, void* out, const 
     return fail(-1, "lv_token_shift: bad arguments");
   dim3 grid(static_cast<unsigned>(T)), block(256);
   const bool vec4 = W % 4 == 0 && aligned16(h) && aligned16(mu) && aligned16(state) && aligned16(out);
+  const bool tiled = vec4 && M <= kShiftMax && T >= 128 * kShiftTile;
+  if (tiled) {
+    dim3 tgrid(static_cast<unsigned>((T + kShiftTile - 1) / kShiftTile), (W / 4 + 255) / 256);
+    if (dtype == LV_MIX_BF16)
+      token_shift_tile_kernel<bf16_t><<<tgrid, block, 0, as_stream(stream)>>>(
+          static_cast<const bf16_t*>(h), static_cast<const float*>(mu), static_cast<bf16_t*>(state), static_cast<bf16_t*>(out), cu_q,
+          ctx_lens, slots, tok_seq, T, W, M);
+    else if (dtype == LV_MIX_F32)
+      token_shift_tile_kernel<float><<<tgrid, block, 0, as_stream(stream)>>>(
+          static_cast<const float*>(h), static_cast<const float*>(mu), static_cast<float*>(state), static_cast<float*>(out), cu_q,
+          ctx_lens, slots, tok_seq, T, W, M);
+    else
+      return fail(-1, "lv_token_shift: dtype %d", dtype);
+    return launched("lv_token_shift");
+  }
 #define LVMIX_SHIFT(TT, VV)                                                                                               \
   token_shift_kernel<TT, VV><<<grid, block, 0, as_stream(stream)>>>(static_cast<const TT*>(h), static_cast<const float*>(mu), \
                                                                    static_cast<TT*>(state), static_cast<TT*>(out), cu_q,  \
@@ -809,6 +912,19 @@ int lv_grouped_gate_norm(const void* o, const void* z, int64_t ldz, const void* 
   const int gs = N / groups;
   const bool vec4 = gs % 4 == 0 && ldz % 4 == 0 && aligned16(o) && aligned8(z) && aligned16(w) && aligned16(out) &&
                     (dtype == LV_MIX_BF16 || aligned16(z));
+  if (vec4 && gs <= 4 * kWave * kPartRegs && (dtype == LV_MIX_BF16 || dtype == LV_MIX_F32)) {
+    const int64_t items = T * groups;
+    dim3 pgrid(static_cast<unsigned>((items + 3) / 4)), pblock(256);
+    if (dtype == LV_MIX_BF16)
+      part_gate_norm_kernel<bf16_t><<<pgrid, pblock, 0, as_stream(stream)>>>(
+          static_cast<const float*>(o), static_cast<const bf16_t*>(z), ldz, static_cast<const float*>(w), static_cast<bf16_t*>(out),
+          items, N, groups, eps);
+    else
+      part_gate_norm_kernel<float><<<pgrid, pblock, 0, as_stream(stream)>>>(
+          static_cast<const float*>(o), static_cast<const float*>(z), ldz, static_cast<const float*>(w), static_cast<float*>(out),
+          items, N, groups, eps);
+    return launched("lv_grouped_gate_norm");
+  }
   dim3 grid(static_cast<unsigned>(T * groups)), block(gs > 512 ? 256 : 64);
 #define LVMIX_GGN(TT, VV)                                                                                                   \
   grouped_gate_norm_kernel<TT, VV><<<grid, block, 0, as_stream(stream)>>>(static_cast<const float*>(o), static_cast<const TT*>(z), ldz, \

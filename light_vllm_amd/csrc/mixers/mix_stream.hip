@@ -487,6 +487,31 @@ __global__ __launch_bounds__(256) void head_norm_gate_kernel(const float* __rest
   }
 }
 
+// Four entries per lane: a head of Dv <= 256 entries sits in P lanes (the power of two at or above Dv / 4), a wave holds 64 / P
+// heads, each value is read once. Taken when head size, row strides and addresses are multiples of four entries.
+template <typename T>
+__global__ __launch_bounds__(256) void vec_head_norm_gate_kernel(const float* __restrict__ o, const T* __restrict__ gate,
+                                                                 int64_t ld_gate, const float* __restrict__ norm_w,
+                                                                 T* __restrict__ out, int64_t items, int H, int Dv, float eps,
+                                                                 int gate_act, int w_ld, const float* __restrict__ den, int P) {
+  const int wave = threadIdx.x / kWave, lane = threadIdx.x % kWave;
+  const int per_wave = kWave / P, e = 4 * (lane % P);
+  const int64_t item = (static_cast<int64_t>(blockIdx.x) * (blockDim.x / kWave) + wave) * per_wave + lane / P;
+  const bool live = item < items && e < Dv;
+  const int64_t t = item / H;
+  const int h = static_cast<int>(item - t * H);
+  float4 v = live ? ld4(o + item * Dv + e) : float4{0.0f, 0.0f, 0.0f, 0.0f};
+  const float f = (live && den != nullptr) ? 1.0f / den[item] : 1.0f;
+  float ss = (v.x * v.x + v.y * v.y) + (v.z * v.z + v.w * v.w);
+  for (int x = P >> 1; x > 0; x >>= 1) ss += __shfl_xor(ss, x, kWave);
+  if (!live) return;
+  const float inv = f / sqrtf(ss * f * f / static_cast<float>(Dv) + eps);
+  const float4 w = ld4(norm_w + static_cast<int64_t>(h) * w_ld + e), g = ld4(gate + t * ld_gate + static_cast<int64_t>(h) * Dv + e);
+  auto act = [&](float x) { return gate_act == LV_MIX_GATE_SILU ? siluf_(x) : sigmoidf_(x); };
+  st4(out + item * Dv + e, float4{v.x * inv * w.x * act(g.x), v.y * inv * w.y * act(g.y), v.z * inv * w.z * act(g.z),
+                                  v.w * inv * w.w * act(g.w)});
+}
+
 // The same for heads of many entries (a norm over a whole row of heads is one such head): one workgroup per (token, head),
 // four entries per thread and access.
 template <typename T>
@@ -680,6 +705,22 @@ int lv_scaled_head_norm_gate(const void* o, const void* den, const void* gate, i
       wide_head_norm_gate_kernel<float><<<wgrid, wblock, 0, as_stream(stream)>>>(
           static_cast<const float*>(o), static_cast<const float*>(gate), ld_gate, static_cast<const float*>(norm_w),
           static_cast<float*>(out), H, Dv, eps, gate_act, w_ld, static_cast<const float*>(den));
+    return launched("lv_head_norm_gate");
+  }
+  if (Dv <= 4 * kWave && Dv % 4 == 0 && ld_gate % 4 == 0 && aligned(o) && aligned(norm_w) && aligned(out) &&
+      (reinterpret_cast<uintptr_t>(gate) & (dtype == LV_MIX_F32 ? 15 : 7)) == 0 && (dtype == LV_MIX_BF16 || dtype == LV_MIX_F32)) {
+    int P = 1;
+    while (4 * P < Dv) P <<= 1;                      // lanes that hold one head
+    const int64_t per_block = 4 * (kWave / P);
+    dim3 vgrid(static_cast<unsigned>((items + per_block - 1) / per_block)), vblock(256);
+    if (dtype == LV_MIX_BF16)
+      vec_head_norm_gate_kernel<bf16_t><<<vgrid, vblock, 0, as_stream(stream)>>>(
+          static_cast<const float*>(o), static_cast<const bf16_t*>(gate), ld_gate, static_cast<const float*>(norm_w),
+          static_cast<bf16_t*>(out), items, H, Dv, eps, gate_act, w_ld, static_cast<const float*>(den), P);
+    else
+      vec_head_norm_gate_kernel<float><<<vgrid, vblock, 0, as_stream(stream)>>>(
+          static_cast<const float*>(o), static_cast<const float*>(gate), ld_gate, static_cast<const float*>(norm_w),
+          static_cast<float*>(out), items, H, Dv, eps, gate_act, w_ld, static_cast<const float*>(den), P);
     return launched("lv_head_norm_gate");
   }
   dim3 grid(static_cast<unsigned>((items + 3) / 4)), block(256);
