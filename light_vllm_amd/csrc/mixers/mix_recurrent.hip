@@ -317,7 +317,7 @@ struct ScanShape {
 };
 
 template <typename T, int KIND, int DR, int NW>
-__global__ __launch_bounds__(NW * 64) void gated_scan_kernel(ScanParams p) {
+__global__ __launch_bounds__(NW * 64, DR > 32 ? 2 : (KIND == kScanRowDecay && DR == 32 ? 3 : 4)) void gated_scan_kernel(ScanParams p) {
   extern __shared__ __attribute__((aligned(16))) float sl[];
   using Shape = ScanShape<KIND, DR, NW>;
   constexpr int DP = Shape::kDP, NT = NW * kWave, CH = Shape::kChunk, SEG = Shape::kSeg, R16 = Shape::kRows16;
