@@ -232,3 +232,86 @@ def forward(tokens, W, cfg, cache_round=None):
         x = layer(x, W, i, spec, eps, cache_round)
         trail.append(x)
     return offset_norm(x, W["final.norm"], eps) @ W["embed"].T, trail
+
+
+# ------------------------------------------------------------------------------ random checkpoints
+def tensor_shapes(cfg) -> dict:
+    """name -> shape of every tensor a checkpoint of this configuration holds. The rank of the decay's thin factors is no part
+    of the configuration: `decay_rank` of a right mixer here, 5 without one."""
+    W = int(cfg["width"])
+    t = {"embed": (int(cfg["vocab"]), W), "pos": (int(cfg["max_positions"]), W), "embed.norm": (W,), "final.norm": (W,)}
+    b = (cfg.get("embedding") or {}).get("bigram")
+    if b:
+        t["bigram"] = (int(b["buckets"]) + 1, W)
+    for i, L in enumerate(cfg["layers"]):
+        p, m = f"l{i}.", L["mixer"]
+        t[p + "norm1"] = (W,)
+        q = p + "mix."
+        if L["type"] == "mlstm":
+            H, D, Dv = m["heads"], m["dim"], m["vdim"]
+            t.update({q + "q": (H * D, W), q + "k": (H * D, W), q + "v": (H * Dv, W), q + "g": (H * Dv, W), q + "o": (W, H * Dv),
+                      q + "norm": (H * Dv,), q + "i": (H, W), q + "i.b": (H,), q + "f": (H, W), q + "f.b": (H,)})
+        elif L["type"] == "mamba2":
+            H, inner, C = m["heads"], m["heads"] * m["vdim"], m["heads"] * m["vdim"] + 2 * m["groups"] * m["state"]
+            t.update({q + "in": (inner + C + H, W), q + "conv": (C, m["conv"]), q + "conv.b": (C,), q + "dt_bias": (H,),
+                      q + "A_log": (H,), q + "D": (H,), q + "norm": (inner,), q + "o": (W, inner)})
+        else:
+            a, r = m["left"], m["right"]
+            H, G, D, Dv = a["heads"], a["kv_heads"], a["dim"], a["vdim"]
+            for nm, n in (("q", H * D), ("k", G * D), ("v", G * Dv)):
+                t.update({q + "left." + nm: (n, W), q + "left." + nm + ".conv": (n, a["conv"])})
+            t.update({q + "left.o": (W, H * Dv), q + "left.out": (W,)})
+            H, n, R = r["heads"], r["heads"] * r["dim"], int(r.get("decay_rank", 5))
+            for c in "rkvgw":
+                t[q + "right.mu." + c] = (W,)
+            for c in "rkvg":
+                t[q + "right." + c] = (n, W)
+            t.update({q + "right.w1": (R, W), q + "right.w2": (n, R), q + "right.w0": (n,), q + "right.u": (H, r["dim"]),
+                      q + "right.norm": (n,), q + "right.o": (W, n), q + "right.out": (W,)})
+        if L.get("mlp") is not None:
+            t.update({p + "norm2": (W,), p + "mlp.up": (L["mlp"]["ff"], W), p + "mlp.down": (W, L["mlp"]["ff"])})
+    return t
+
+
+def random_weights(cfg, seed: int) -> dict:
+    """A seeded checkpoint, float64 values that bfloat16 holds exactly. Scales keep activations of order one and make the
+    hashed pairs, the positions, the old taps, the shifted inputs, the gates and the skips all matter, with states that remember
+    for tens to hundreds of tokens."""
+    g = torch.Generator().manual_seed(seed)
+    scale = float((cfg.get("embedding") or {}).get("scale", 1.0))
+    out = {}
+    for name, shape in tensor_shapes(cfg).items():
+        leaf = name.rsplit(".", 1)[-1]
+        x = torch.randn(tuple(shape), generator=g)
+        if name in ("embed.norm", "final.norm") or leaf in ("norm1", "norm2"):
+            x = 0.3 * x
+        elif leaf in ("norm", "out"):
+            x = 1.0 + 0.3 * x
+        elif name == "embed":
+            x = x / max(scale, 1.0)
+        elif name in ("bigram", "pos"):
+            x = 0.7 * x
+        elif name.endswith(".f.b"):
+            x = 2.5 + 1.5 * x
+        elif name.endswith(".i.b"):
+            x = -0.5 + x
+        elif name.endswith("conv.b"):
+            x = 0.3 * x
+        elif leaf in ("i", "f"):
+            x = 1.5 * x / shape[-1] ** 0.5
+        elif leaf == "w0":
+            x = -2.5 + 1.5 * x
+        elif leaf == "dt_bias":
+            x = -2.0 + x
+        elif leaf == "A_log":
+            x = 0.7 * x
+        elif leaf in ("D", "u") or ".mu." in name:
+            x = 0.5 + 0.4 * x
+        elif leaf == "conv":
+            x = x / shape[-1] ** 0.5
+        elif ".left." in name and leaf in ("q", "k"):
+            x = 1.7 * x / shape[-1] ** 0.5
+        else:
+            x = x / shape[-1] ** 0.5
+        out[name] = x.to(torch.bfloat16).to(F64)
+    return out

@@ -1,0 +1,75 @@
+"""Feditar on the CPU: the engine's host logic (ragged scheduling, pages, state slots, checkpoint placement) with the
+package's torch restatement of the kernels, against the oracle."""
+import pytest
+
+from tests import _feditar as K
+from tests import _feditar_cases as C
+
+DEV = "cpu"
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_mechanisms(dtype):
+    C.case_embed(DEV, dtype)
+    C.case_causal_conv(DEV, dtype)
+    C.case_conv_qkv_store(DEV, dtype)
+    C.case_token_shift(DEV, dtype)
+    C.case_norms_and_acts(DEV, dtype)
+
+
+@pytest.mark.parametrize("case", [C.case_scan_step, C.case_scan_log_gates, C.case_scan_row_decay], ids=["step", "log_gates", "row_decay"])
+def test_scans(case, monkeypatch):
+    monkeypatch.setattr(C, "MANY", C.SCAN_SIZES[0])
+    case(DEV, "float32")
+
+
+def test_capped_attention():
+    C.case_capped_attention(DEV, "float32")
+
+
+def test_checkpoint_placement(tmp_path):
+    C.case_checkpoint_placement(tmp_path)
+
+
+@pytest.mark.parametrize("name", ["CFG_MAIN", "CFG_ODD", "CFG_WIDE"])
+def test_layer_by_layer(tmp_path, name):
+    C.case_layer_by_layer(DEV, tmp_path, cfg=getattr(K, name))
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_engine_schedules(tmp_path, dtype):
+    C.case_engine_schedules(DEV, dtype, tmp_path)
+
+
+@pytest.mark.parametrize("name", ["CFG_ODD", "CFG_WIDE", "CFG_ONE", "CFG_ONE_MEM"])
+def test_engine_other_sizes(tmp_path, name):
+    C.case_engine_schedules(DEV, "float32", tmp_path, cfg=getattr(K, name), seed=9)
+
+
+@pytest.mark.parametrize("seed", [201, 204])
+def test_engine_random_configs(tmp_path, seed):
+    C.case_engine_random_config(DEV, "float32", tmp_path, seed)
+
+
+def test_engine_long(tmp_path):
+    C.case_engine_long(DEV, "float32", tmp_path)
+
+
+def test_engine_far_token(tmp_path):
+    C.case_engine_far_token(DEV, tmp_path)
+
+
+def test_engine_reuse_of_pages_and_slots(tmp_path):
+    C.case_engine_reuse(DEV, "float32", tmp_path)
+
+
+def test_engine_long_decode(tmp_path):
+    C.case_engine_long_decode(DEV, "float32", tmp_path)
+
+
+def test_position_limit(tmp_path):
+    C.case_position_limit(DEV, tmp_path)
+
+
+def test_generate(tmp_path):
+    C.case_generate(DEV, tmp_path)

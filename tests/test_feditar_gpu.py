@@ -1,0 +1,84 @@
+"""Feditar on the GPU: the HIP kernels of liblvmix.so, alone and through the engine, against the oracle."""
+import pytest
+
+from tests import _feditar as K
+from tests import _feditar_cases as C
+
+pytestmark = pytest.mark.gpu
+DEV = "cuda"
+DTYPES = ["float32", "bfloat16"]
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("case", [C.case_embed, C.case_causal_conv, C.case_conv_qkv_store, C.case_token_shift, C.case_scan_step,
+                                  C.case_scan_log_gates, C.case_scan_row_decay, C.case_norms_and_acts, C.case_capped_attention],
+                         ids=lambda c: c.__name__[5:])
+def test_mechanism(gpu, case, dtype):
+    case(DEV, dtype)
+
+
+def test_matrix_core_attention_agrees_with_the_vector_kernel(gpu):
+    """The same bf16 cases with the vector kernel forced: both kernels cap the same scores."""
+    from light_vllm_amd import mix_ops
+    old, mix_ops.WINDOW_ATTN_KERNEL = mix_ops.WINDOW_ATTN_KERNEL, "valu"
+    try:
+        C.case_capped_attention(DEV, "bfloat16")
+    finally:
+        mix_ops.WINDOW_ATTN_KERNEL = old
+
+
+@pytest.mark.parametrize("name", ["CFG_MAIN", "CFG_ODD", "CFG_WIDE"])
+def test_layer_by_layer(gpu, tmp_path, name):
+    C.case_layer_by_layer(DEV, tmp_path, cfg=getattr(K, name))
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_engine_schedules(gpu, tmp_path, dtype):
+    C.case_engine_schedules(DEV, dtype, tmp_path)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name", ["CFG_ODD", "CFG_WIDE", "CFG_ONE", "CFG_ONE_MEM"])
+def test_engine_other_sizes(gpu, tmp_path, name, dtype):
+    C.case_engine_schedules(DEV, dtype, tmp_path, cfg=getattr(K, name), seed=9)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("seed", [201, 202, 203, 204, 205, 206])
+def test_engine_random_configs(gpu, tmp_path, seed, dtype):
+    C.case_engine_random_config(DEV, dtype, tmp_path, seed)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_engine_long(gpu, tmp_path, dtype):
+    C.case_engine_long(DEV, dtype, tmp_path)
+
+
+def test_engine_far_token(gpu, tmp_path):
+    C.case_engine_far_token(DEV, tmp_path)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_engine_reuse_of_pages_and_slots(gpu, tmp_path, dtype):
+    C.case_engine_reuse(DEV, dtype, tmp_path)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_engine_long_decode(gpu, tmp_path, dtype):
+    C.case_engine_long_decode(DEV, dtype, tmp_path)
+
+
+def test_position_limit(gpu, tmp_path):
+    C.case_position_limit(DEV, tmp_path)
+
+
+def test_generate(gpu, tmp_path):
+    C.case_generate(DEV, tmp_path)
+
+
+def test_generate_from_graphs(gpu, tmp_path):
+    C.case_generate(DEV, tmp_path, enforce_eager=False)
+
+
+def test_generate_bf16_graphs_like_eager(gpu, tmp_path):
+    C.case_generate_bf16_graphs_like_eager(DEV, tmp_path)

@@ -61,3 +61,26 @@ def test_argument_validation_happens_before_any_launch():
     assert lib.lv_moe_grouped_glu_ff(p, p, p, p, p, 0, p, p, 1, 48, 32, 4, 2, 1.0, 1.702, None) == -1     # width no multiple of 32
     assert lib.lv_moe_grouped_glu_ff(p, p, p, p, p, 100, p, p, 1, 64, 32, 4, 2, 1.0, 1.702, None) == -1   # down rows shorter than E*F
     assert lib.lv_window_pool_attn(p, p, p, None, None, p, 4, p, p, p, p, p, 1, 1, 4, 2, 8, 8, 16, 64, 0, 0.5, 0, 0, 0, 5, 0, None) == -1   # gate kind
+    # scans, convolutions and the steps around them
+    assert lib.lv_causal_conv(None, 0, None, None, None, None, None, None, None, 0, 5, 8, 4, 1, 0, None) == 0           # no sequence
+    conv = lambda **kw: [p, kw.get("ld", 8), p, None, kw.get("state", p), p, p, p, p, 1, 1, 8, kw.get("taps", 4), 1, kw.get("dt", 0), None]  # noqa: E731
+    assert lib.lv_causal_conv(*conv(ld=7)) == -1 and lib.lv_causal_conv(*conv(taps=0)) == -1
+    assert lib.lv_causal_conv(*conv(state=None)) == -1 and lib.lv_causal_conv(*conv(dt=9)) == -1
+    qkv = lambda **kw: [p, kw.get("ld", 64), p, p, p, p, p, p, p, p, p, 1, 1, 1, kw.get("H", 4), kw.get("G", 2), 8, 8, 3, kw.get("coef", 0.5),  # noqa: E731
+                        kw.get("every", 4), 16, 0, None]
+    assert lib.lv_conv_qkv_store(*qkv(H=3)) == -1 and lib.lv_conv_qkv_store(*qkv(ld=63)) == -1 and lib.lv_conv_qkv_store(*qkv(every=0)) == -1
+    scan = lambda **kw: [kw.get("kind", 0), p, kw.get("ldq", 16), p, 16, p, 16, p, kw.get("a2", p), kw.get("lda", 16), p, p, kw.get("p2", p), 1.0,  # noqa: E731
+                         kw.get("cap", 1.0), p, kw.get("ns", p), p, p, p, p, p, p, 1, kw.get("H", 2), kw.get("G", 2), kw.get("D", 8), 8, 0, None]
+    assert lib.lv_gated_scan(*scan(kind=5)) == -1 and lib.lv_gated_scan(*scan(p2=None)) == -1
+    assert lib.lv_gated_scan(*scan(kind=1, ns=None)) == -1 and lib.lv_gated_scan(*scan(kind=1, cap=0.0)) == -1
+    assert lib.lv_gated_scan(*scan(kind=2, G=1)) == -1 and lib.lv_gated_scan(*scan(kind=2, lda=15)) == -1
+    assert lib.lv_gated_scan(*scan(ldq=15)) == -1 and lib.lv_gated_scan(*scan(H=3)) == -1
+    assert lib.lv_gated_scan(*scan(G=1, D=257, ldq=512)) in (-1, -2)
+    assert lib.lv_token_shift(p, p, None, p, p, p, p, p, 1, 8, 5, 0, None) == -1
+    assert lib.lv_grouped_gate_norm(p, p, 8, p, p, 1, 8, 3, 1e-6, 0, None) == -1                                      # parts that do not divide
+    assert lib.lv_scaled_head_norm_gate(p, None, p, 16, p, 5, p, 1, 2, 8, 1e-6, 0, 0, None) == -1                      # weight stride
+    assert lib.lv_residual_pair_norm(p, p, p, p, None, 0.5, 1e-6, p, 1.0, p, 1, 8, 1e-6, 0, None) == -1
+    assert lib.lv_embed_norm(p, p, 8, 1.0, p, 0, 1, 1, p, None, 0, p, p, 1.0, 1e-6, p, p, p, p, p, p, 1, 8, 0, None) == -1   # no buckets
+    assert lib.lv_embed_norm(p, p, 8, 1.0, None, 0, 0, 0, None, p, 0, p, p, 1.0, 1e-6, p, p, p, p, p, p, 1, 8, 0, None) == -1   # empty position table
+    assert lib.lv_unary_act(p, p, 8, 17, 0, None) == -1
+    assert lib.lv_masked_attn(p, p, p, None, None, None, 0, p, p, p, p, p, 1, 1, 4, 2, 8, 8, 16, 64, 0, 0, 0, 0.5, -1.0, 0, None, 0, 0, 1, 0, None) == -1   # cap
