@@ -7,7 +7,7 @@ set -e
 cd "$(dirname "$0")/../light_vllm_amd/csrc"
 mkdir -p ../../tools/abl
 for mask in "$@"; do
-  /opt/rocm/bin/hipcc -O3 -std=c++17 -fPIC --offload-arch=gfx950 -I../../include -I. -w -DLV_DECODE_ABL=$mask -shared \
+  /opt/rocm/bin/hipcc -O3 -std=c++17 -fPIC --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops -I../../include -I. -w -DLV_DECODE_ABL=$mask -shared \
     api.hip store_kvcache.hip fused_ops.hip decode_attn.hip prefill_attn.hip comm.hip -o ../../tools/abl/liblvattn_abl$mask.so &
 done
 wait

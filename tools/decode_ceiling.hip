@@ -4,7 +4,7 @@
 // block table entry -> first row address, three dependent loads), the epilogue (LDS exchange,
 // barrier, output store). Average of 30 back-to-back launches that alternate between two cache
 // sets (2 GiB each, far beyond the 256 MiB last-level cache), not the best single launch.
-// Build: hipcc -O3 --offload-arch=gfx950 tools/decode_ceiling.hip -o tools/decode_ceiling
+// Build: hipcc -O3 --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops tools/decode_ceiling.hip -o tools/decode_ceiling
 #include <hip/hip_runtime.h>
 #include <stdio.h>
 #include <stdint.h>

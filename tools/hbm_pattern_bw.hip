@@ -1,7 +1,7 @@
 // Ceiling of the paged-decode ACCESS PATTERN with no arithmetic: workgroup (sequence, kv head) reads
 // the 256-byte rows of its head for every token of the sequence (stride Hkv*256 B) from a K and a
 // V cache; one wave instruction = 4 tokens x 16 lanes x 16 B. Same grid/shape as bench.py's config.
-// Build: hipcc -O3 --offload-arch=gfx950 tools/hbm_pattern_bw.hip -o tools/hbm_pattern_bw
+// Build: hipcc -O3 --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops tools/hbm_pattern_bw.hip -o tools/hbm_pattern_bw
 #include <hip/hip_runtime.h>
 #include <stdio.h>
 #include <stdint.h>

@@ -1,6 +1,6 @@
 // Read-only HBM streaming ceiling on this device: every lane issues U independent 16-byte
 // non-temporal loads per iteration over a buffer far larger than the 256 MiB last-level cache.
-// Build: hipcc -O3 --offload-arch=gfx950 tools/hbm_read_bw.hip -o tools/hbm_read_bw
+// Build: hipcc -O3 --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops tools/hbm_read_bw.hip -o tools/hbm_read_bw
 #include <hip/hip_runtime.h>
 #include <stdio.h>
 #include <stdint.h>

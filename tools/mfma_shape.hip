@@ -4,7 +4,7 @@
 // milliseconds per launch; reports TFLOP/s from the wall time of the launch and the shader clock
 // the waves saw (s_memtime ticks per 100 MHz s_memrealtime tick). The spec peak (2.5 PFLOP/s) is
 // 1024 SIMDs x 1024 FLOP per cycle x 2.4 GHz; this measures the clock the chip keeps under that load.
-//   hipcc -O3 --offload-arch=gfx950 tools/mfma_shape.hip -o tools/mfma_shape && tools/mfma_shape 1 1 1
+//   hipcc -O3 --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops tools/mfma_shape.hip -o tools/mfma_shape && tools/mfma_shape 1 1 1
 #include <hip/hip_runtime.h>
 #include <stdio.h>
 typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;

@@ -1,6 +1,6 @@
 // Diagnostic harness (not shipped): builds the prefill kernel with s_memtime stamps and prints the
 // share of wave time spent in each loop segment. Build and run:
-//   hipcc -O3 -std=c++17 --offload-arch=gfx950 -DLV_STAMPS -Iinclude -Ilight_vllm_amd/csrc \
+//   hipcc -O3 -std=c++17 --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops -DLV_STAMPS -Iinclude -Ilight_vllm_amd/csrc \
 //         tools/prefill_diag.hip -o tools/prefill_diag && tools/prefill_diag [seqlen [kernel_hint [heads kv_heads]]]
 // kernel_hint: an LV_PREFILL_KERNEL_* value (0 = the library's choice, 3 = phase-locked, 5 = 64 rows per wave).
 #include <stdarg.h>

@@ -1,7 +1,7 @@
 // Diagnostic harness (not shipped): the life of the phase-locked prefill kernel's workgroups on a compute
 // unit - prologue (Q fragments, first K/V tiles), tile loop, epilogue (output stores), and the gap until
 // the next workgroup starts on the same compute unit. Build and run:
-//   hipcc -O3 -std=c++17 --offload-arch=gfx950 -DLV_TIMELINE -Iinclude -Ilight_vllm_amd/csrc \
+//   hipcc -O3 -std=c++17 --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops -DLV_TIMELINE -Iinclude -Ilight_vllm_amd/csrc \
 //         tools/prefill_timeline.hip -o tools/prefill_timeline && tools/prefill_timeline [seqlen [heads kv_heads [persistent]]]
 #include <stdarg.h>
 #include <stdio.h>
