@@ -37,7 +37,10 @@
 #include <stdio.h>
 #include <string.h>
 
+#include <mutex>
 #include <new>
+#include <utility>
+#include <vector>
 
 #include "lv_comm.h"
 #include "lv_common.h"
@@ -324,6 +327,27 @@ struct lv_comm {
   int* host_failed_dev = nullptr;                      // its device pointer
 };
 
+// Uncached allocations are not handed back to the driver before the process ends (memory allocated after such a free has held
+// wrong values): a destroyed communicator leaves its allocation here for the next one on the same device.
+static std::mutex g_idle_lock;
+static std::vector<std::pair<int, unsigned char*>> g_idle;
+
+static unsigned char* take_idle(int device) {
+  std::lock_guard<std::mutex> hold(g_idle_lock);
+  for (size_t i = 0; i < g_idle.size(); ++i)
+    if (g_idle[i].first == device) {
+      unsigned char* p = g_idle[i].second;
+      g_idle.erase(g_idle.begin() + static_cast<long>(i));
+      return p;
+    }
+  return nullptr;
+}
+
+static void leave_idle(int device, unsigned char* p) {
+  std::lock_guard<std::mutex> hold(g_idle_lock);
+  g_idle.emplace_back(device, p);
+}
+
 #define LV_HIP_OK(call, what)                                                                   \
   do {                                                                                          \
     hipError_t e_ = (call);                                                                     \
@@ -352,7 +376,7 @@ int lv_comm_create(int rank, int world_size, int timeout_ms, lv_comm_t** comm) {
   int rc = LV_OK;
   do {
     hipError_t e = hipGetDevice(&c->device);
-    if (e == hipSuccess)
+    if (e == hipSuccess && (c->mine = take_idle(c->device)) == nullptr)
       e = hipExtMallocWithFlags(reinterpret_cast<void**>(&c->mine), kCommAllocBytes, hipDeviceMallocUncached);
     if (e == hipSuccess) e = hipMemset(c->mine, 0, kCommAllocBytes);
     if (e == hipSuccess) e = hipMalloc(reinterpret_cast<void**>(&c->epoch), kCommMaxBlocks * sizeof(uint32_t) + 256);
@@ -371,7 +395,7 @@ int lv_comm_create(int rank, int world_size, int timeout_ms, lv_comm_t** comm) {
     c->base[rank] = c->mine;
   } while (0);
   if (rc != LV_OK) {
-    if (c->mine) (void)hipFree(c->mine);
+    if (c->mine) leave_idle(c->device, c->mine);
     if (c->epoch) (void)hipFree(c->epoch);
     if (c->host_failed) (void)hipHostFree(c->host_failed);
     delete c;
@@ -561,7 +585,7 @@ int lv_comm_destroy(lv_comm_t* c) {
   (void)hipDeviceSynchronize();
   for (int r = 0; r < c->world; ++r)
     if (r != c->rank && c->base[r]) (void)hipIpcCloseMemHandle(c->base[r]);
-  if (c->mine) (void)hipFree(c->mine);
+  if (c->mine) leave_idle(c->device, c->mine);
   if (c->epoch) (void)hipFree(c->epoch);
   if (c->host_failed) (void)hipHostFree(c->host_failed);
   delete c;

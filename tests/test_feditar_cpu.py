@@ -73,3 +73,7 @@ def test_position_limit(tmp_path):
 
 def test_generate(tmp_path):
     C.case_generate(DEV, tmp_path)
+
+
+def test_generate_under_preemption(tmp_path):
+    C.case_generate_preemption(DEV, tmp_path)

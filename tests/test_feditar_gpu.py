@@ -82,3 +82,7 @@ def test_generate_from_graphs(gpu, tmp_path):
 
 def test_generate_bf16_graphs_like_eager(gpu, tmp_path):
     C.case_generate_bf16_graphs_like_eager(DEV, tmp_path)
+
+
+def test_generate_under_preemption(gpu, tmp_path):
+    C.case_generate_preemption(DEV, tmp_path)
