@@ -1369,7 +1369,7 @@ def _feditar_kernel_table(z, fz, sz, dev, batch, prompt_len):
         gi, gf = mproj[:, 4 * Hm * D:4 * Hm * D + Hm], mproj[:, 4 * Hm * D + Hm:]
         ib, fb = torch.zeros(Hm, device=dev), torch.full((Hm,), 3.0, device=dev)
         S1 = torch.zeros(B, Hm, D, D, device=dev)
-        n1, m1 = torch.zeros(B, Hm, D, device=dev), torch.zeros(B, Hm, -(-D // 64), device=dev)
+        n1, m1 = torch.zeros(B, Hm, D, device=dev), torch.zeros(B, Hm, mix_ops.scan_copies(D), device=dev)
         add("gated_scan, log gates (matrix memory)", phase,
             lambda: mix_ops.gated_scan(mix_ops.SCAN_LOG_GATES, mq, mk, mv, gi, ib, fb, step, S1, Hm, Hm, D, D, a2=gf, q_scale=D ** -0.5,
                                        cap=15.0, norm_state=n1, max_state=m1), **scan_work(Hm, D, D, Hm * D * 10))

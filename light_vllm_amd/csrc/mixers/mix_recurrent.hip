@@ -22,6 +22,10 @@ namespace lvmix {
 
 __device__ __forceinline__ float log_sigmoidf_(float x) { return x < 0.0f ? x - log1pf(expf(x)) : -log1pf(expf(-x)); }
 
+__device__ __forceinline__ float read_lane(float x, int i) {           // i uniform over the wave
+  return __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, x), i));
+}
+
 __device__ __forceinline__ float block_sum(float a, float* red) {      // over the workgroup's waves (at most four)
   a = wave_sum(a);
   const int waves = blockDim.x / kWave;
@@ -302,17 +306,54 @@ struct ScanParams {
   int H, G, D, Dv;
 };
 
-// NW waves a workgroup, DR = rows of the state each wave owns (NW * DR >= D; rows beyond D stay zero); lane = value column.
+// N consecutive f32 values from LDS, N = 1, 2 or a multiple of 4 (aligned to as many).
+template <int N>
+__device__ __forceinline__ void lds_rows(const float* p, float (&v)[N]) {
+  if constexpr (N % 4 == 0) {
+#pragma unroll
+    for (int r = 0; r < N; r += 4) {
+      const float4 x = *reinterpret_cast<const float4*>(p + r);
+      v[r] = x.x; v[r + 1] = x.y; v[r + 2] = x.z; v[r + 3] = x.w;
+    }
+  } else if constexpr (N == 2) {
+    const float2 x = *reinterpret_cast<const float2*>(p);
+    v[0] = x.x; v[1] = x.y;
+  } else {
+    v[0] = p[0];
+  }
+}
+
+template <int CTRL>
+__device__ __forceinline__ float quad_perm(float x) {
+  return __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, x), CTRL, 0xf, 0xf, true));
+}
+// Four lanes hold shares of four columns each; lane rl of the four is left with the sum of column rl.
+__device__ __forceinline__ float quad_columns(const float (&p)[4], int rl) {
+  const bool odd = rl & 1, high = rl & 2;
+  const float a = (odd ? p[1] : p[0]) + quad_perm<0xb1>(odd ? p[0] : p[1]);     // columns 0 | 1 over lanes rl, rl ^ 1
+  const float b = (odd ? p[3] : p[2]) + quad_perm<0xb1>(odd ? p[2] : p[3]);     // columns 2 | 3
+  return (high ? b : a) + quad_perm<0x4e>(high ? a : b);
+}
+
+// NW waves a workgroup on 64 value columns, DR = rows of the state each wave owns (NW * DR >= D; rows beyond D stay zero). A lane
+// holds a block of DR / 4 rows by 4 columns: four neighbouring lanes share the columns and divide the wave's rows, so that a
+// token costs a lane DR / 4 keys, DR / 4 queries and 4 values from LDS for DR entries (with a lane per column every lane reads
+// all DR keys and queries, and the kernel ran at the speed of those reads), and the four lanes' read-outs meet in the ALU.
 // A chunk of tokens is fetched into registers one chunk ahead and staged in LDS; every wave then walks the chunk alone (its
 // rows of S need nobody else's) and leaves its share of each read-out in LDS; the shares are added when the chunk is done.
+//
+// Where a head has one decay per token, S is held as F S' with a number F that takes the decays: S' <- S' + (write / F) k v^T,
+// o = F S'^T q, two multiply-adds per entry and token instead of a multiply more. Before F would fall below kMinFactor it is
+// multiplied into S' and starts again at 1, so nothing but exponents differs from the plain recurrence.
+constexpr float kMinFactor = 1.0f / (1 << 30);
+
 template <int KIND, int DR, int NW>
 struct ScanShape {
   static constexpr int kDP = NW * DR;
   static constexpr int kChunk = kDP >= 256 ? 8 : 16;
   static constexpr int kSeg = kDP > kWave ? kDP / kWave : 1;         // partial sums of a token's bonus
-  static constexpr int kRows16 = DR > 16 ? DR / 16 : 1;              // a wave's shares of the normaliser's read-out per token
-  static constexpr int kExtra = KIND == kScanStep ? 0 : (KIND == kScanRowDecay ? kChunk * kDP : kChunk * NW * kRows16);
-  static constexpr size_t kLds = sizeof(float) * (2 * kChunk * kDP + kChunk * kWave + kChunk * NW * kWave + kExtra + 4 * kChunk +
+  static constexpr int kExtra = KIND == kScanStep ? 0 : (KIND == kScanRowDecay ? kChunk * kDP : kChunk * kDP / 16);
+  static constexpr size_t kLds = sizeof(float) * (2 * kChunk * kDP + kChunk * kWave + kChunk * NW * kWave + kExtra + 8 * kChunk +
                                                   kChunk * kSeg);
 };
 
@@ -320,36 +361,56 @@ template <typename T, int KIND, int DR, int NW>
 __global__ __launch_bounds__(NW * 64, DR > 32 ? 2 : (KIND == kScanRowDecay && DR == 32 ? 3 : 4)) void gated_scan_kernel(ScanParams p) {
   extern __shared__ __attribute__((aligned(16))) float sl[];
   using Shape = ScanShape<KIND, DR, NW>;
-  constexpr int DP = Shape::kDP, NT = NW * kWave, CH = Shape::kChunk, SEG = Shape::kSeg, R16 = Shape::kRows16;
+  constexpr int DP = Shape::kDP, NT = NW * kWave, CH = Shape::kChunk, SEG = Shape::kSeg;
   float* k_lds = sl;                               // [CH][DP]
   float* q_lds = k_lds + CH * DP;                  // [CH][DP]
-  float* x_lds = q_lds + CH * DP;                  // [CH][DP] row decays, or [CH][NW * R16] normaliser shares
+  float* x_lds = q_lds + CH * DP;                  // [CH][DP] row decays, or [CH][DP / 16] normaliser shares
   float* v_lds = x_lds + Shape::kExtra;            // [CH][64]
   float* part_o = v_lds + CH * kWave;              // [CH][NW][64]
-  float* sc_lds = part_o + CH * NW * kWave;        // [CH][4]: decay, write, floor of the normaliser
-  float* bon_lds = sc_lds + 4 * CH;                // [CH][SEG]
+  float* sc_all = part_o + CH * NW * kWave;        // [2][CH][4]: what S' is multiplied by, write / F, F, floor of the normaliser
+  float* bon_lds = sc_all + 8 * CH;                // [CH][SEG]
   const int lane = threadIdx.x % kWave, rp = threadIdx.x / kWave;
-  const int col = blockIdx.x * kWave + lane;
+  constexpr int RL = DR / 4;                       // rows of a lane's block
+  const int rl = lane & 3;
+  const int col0 = blockIdx.x * kWave + (lane & ~3);
   const int h = blockIdx.y, b = blockIdx.z;
   const int g = h / (p.H / p.G);
   const int q0 = p.cu_q[b], n = p.cu_q[b + 1] - q0;
   if (n <= 0) return;
-  const bool live = col < p.Dv;
-  const int row0 = rp * DR;
+  const int row0 = rp * DR, own0 = row0 + rl * RL;
   const int64_t head = static_cast<int64_t>(p.slots[b]) * p.H + h;
   float* sbase = p.state + head * p.D * p.Dv;
   const bool carry = p.ctx_lens[b] > 0;
-  float s[DR];
+  float s[RL][4];
+  const bool whole = (p.Dv & 3) == 0 && col0 + 3 < p.Dv;               // the block's rows are aligned and inside
 #pragma unroll
-  for (int r = 0; r < DR; ++r)
-    s[r] = (carry && live && row0 + r < p.D) ? sbase[static_cast<int64_t>(row0 + r) * p.Dv + col] : 0.0f;
-  // kScanLogGates: the normaliser's rows lie in the lanes of their wave; one workgroup of a head keeps and reads it. The running
-  // maximum is a copy per workgroup (its place in max_state), so that none waits for another.
+  for (int r = 0; r < RL; ++r)
+#pragma unroll
+    for (int c = 0; c < 4; ++c) s[r][c] = 0.0f;
+  if (carry && whole) {                            // all of a lane's loads in flight at once
+#pragma unroll
+    for (int r = 0; r < RL; ++r) {
+      const float4 x = ld4(sbase + static_cast<int64_t>(min(own0 + r, p.D - 1)) * p.Dv + col0);
+      const bool in = own0 + r < p.D;
+      s[r][0] = in ? x.x : 0.0f; s[r][1] = in ? x.y : 0.0f; s[r][2] = in ? x.z : 0.0f; s[r][3] = in ? x.w : 0.0f;
+    }
+  } else if (carry) {
+#pragma unroll
+    for (int r = 0; r < RL; ++r)
+#pragma unroll
+      for (int c = 0; c < 4; ++c)
+        if (own0 + r < p.D && col0 + c < p.Dv) s[r][c] = sbase[static_cast<int64_t>(own0 + r) * p.Dv + col0 + c];
+  }
+  // kScanLogGates: the first workgroup of a head keeps the normaliser, a row a thread of its last waves. The running maximum is a
+  // copy per workgroup (its place in max_state), so that none waits for another.
   const bool owner = KIND == kScanLogGates && blockIdx.x == 0;
-  const bool nrow = owner && lane < DR && row0 + lane < p.D;
-  float nstate = (nrow && carry) ? p.norm_state[head * p.D + row0 + lane] : 0.0f;
+  const int nr = static_cast<int>(threadIdx.x) - (NT - DP);
+  const bool nrow = owner && nr >= 0 && nr < p.D;
+  float nstate = (nrow && carry) ? p.norm_state[head * p.D + nr] : 0.0f;
   float* mplace = KIND == kScanLogGates ? p.max_state + head * gridDim.x + blockIdx.x : nullptr;
   float m = (KIND == kScanLogGates && carry) ? *mplace : 0.0f;
+
+  float factor = 1.0f, last_factor = 1.0f;         // F: the first wave's running value, and what it ends with
 
   const T* qp = static_cast<const T*>(p.q) + static_cast<int64_t>(g) * p.D;
   const T* kp = static_cast<const T*>(p.k) + static_cast<int64_t>(g) * p.D;
@@ -357,6 +418,10 @@ __global__ __launch_bounds__(NW * 64, DR > 32 ? 2 : (KIND == kScanRowDecay && DR
   const T* ap = static_cast<const T*>(p.a);
   const int d_own = threadIdx.x % DP;              // DP divides the workgroup: a thread stages one row index of every token
   const bool d_in = d_own < p.D;
+  const int tok_own = threadIdx.x / DP;
+  const uint32_t koff = static_cast<uint32_t>(tok_own * static_cast<int>(p.ldk) + d_own);
+  const uint32_t qoff = static_cast<uint32_t>(tok_own * static_cast<int>(p.ldq) + d_own);
+  const uint32_t aoff = static_cast<uint32_t>(tok_own * static_cast<int>(p.lda) + d_own);
   float u_own = 0.0f, w0_own = 0.0f, gate_a = 0.0f, gate_b = 0.0f, skip = 0.0f;
   if (KIND == kScanRowDecay && d_in) {
     w0_own = p.p0[h * p.D + d_own];
@@ -378,13 +443,13 @@ __global__ __launch_bounds__(NW * 64, DR > 32 ? 2 : (KIND == kScanRowDecay && DR
     const int cn = min(CH, n - c0);
     const int64_t tb = static_cast<int64_t>(q0) + c0;
 #pragma unroll
-    for (int it = 0; it < NKQ; ++it) {
-      const int tok = (threadIdx.x + it * NT) / DP;
-      const bool in = tok < cn && d_in;
-      const int64_t t = tb + tok;
-      kreg[it] = in ? ldf(kp + t * p.ldk + d_own) : 0.0f;
-      qreg[it] = in ? ldf(qp + t * p.ldq + d_own) : 0.0f;
-      if (KIND == kScanRowDecay) wreg[it] = in ? ldf(ap + t * p.lda + h * p.D + d_own) : 0.0f;
+    for (int it = 0; it < NKQ; ++it) {             // uniform part of the address per step, a thread's own part once
+      constexpr int per = NT / DP;
+      const int64_t t = tb + it * per;
+      const bool in = tok_own + it * per < cn && d_in;
+      kreg[it] = in ? ldf(kp + t * p.ldk + koff) : 0.0f;
+      qreg[it] = in ? ldf(qp + t * p.ldq + qoff) : 0.0f;
+      if (KIND == kScanRowDecay) wreg[it] = in ? ldf(ap + h * p.D + t * p.lda + aoff) : 0.0f;
     }
 #pragma unroll
     for (int it = 0; it < NV; ++it) {
@@ -398,9 +463,47 @@ __global__ __launch_bounds__(NW * 64, DR > 32 ? 2 : (KIND == kScanRowDecay && DR
       if (KIND == kScanLogGates) breg = ldf(static_cast<const T*>(p.a2) + t * p.lda + h);
     }
   };
+  // Decays and writes of a chunk of cn tokens, lane = token: the first wave's job, done for the next chunk while the last waves are
+  // at the normaliser.
+  auto scalars = [&](int cn, float* sc) {
+    float dec, write, floor_ = 0.0f;
+    if (KIND == kScanStep) {
+      write = softplusf_(areg + gate_a);
+      dec = expf(gate_b * write);
+    } else {
+      const float li = p.cap * tanhf((areg + gate_a) / p.cap);
+      const float lf = log_sigmoidf_(p.cap * tanhf((breg + gate_b) / p.cap));
+      float before = 0.0f, after = 0.0f;         // the running maximum on either side of this lane's token
+      for (int i = 0; i < cn; ++i) {
+        const float nm = fmaxf(read_lane(lf, i) + m, read_lane(li, i));
+        if (lane == i) {
+          before = m;
+          after = nm;
+        }
+        m = nm;
+      }
+      dec = expf(lf + before - after);
+      write = expf(li - after);
+      floor_ = expf(-after);
+    }
+    float mul = 1.0f, fac = 1.0f;
+    for (int i = 0; i < cn; ++i) {
+      const float nf = factor * read_lane(dec, i);
+      const bool fold = nf < kMinFactor;
+      factor = fold ? 1.0f : nf;
+      if (lane == i) {
+        mul = fold ? nf : 1.0f;
+        fac = factor;
+      }
+    }
+    if (lane < CH) *reinterpret_cast<float4*>(sc + lane * 4) = float4{mul, write / fac, fac, floor_};
+  };
   fetch(0);
-  for (int c0 = 0; c0 < n; c0 += CH) {
+  if (KIND != kScanRowDecay && rp == 0) scalars(min(CH, n), sc_all);
+  int buf = 0;
+  for (int c0 = 0; c0 < n; c0 += CH, buf ^= 1) {
     const int cn = min(CH, n - c0);
+    const float* sc_lds = sc_all + buf * 4 * CH;
     // every wave is past the previous chunk's use of what is written here: behind the barrier that followed its token loop
 #pragma unroll
     for (int it = 0; it < NKQ; ++it) {
@@ -420,74 +523,49 @@ __global__ __launch_bounds__(NW * 64, DR > 32 ? 2 : (KIND == kScanRowDecay && DR
 #pragma unroll
     for (int it = 0; it < NV; ++it)
       if (threadIdx.x + it * NT < CH * kWave) v_lds[threadIdx.x + it * NT] = vreg[it];
-    if (KIND == kScanStep && threadIdx.x < CH) {
-      const float dt = softplusf_(areg + gate_a);
-      sc_lds[threadIdx.x * 4] = expf(gate_b * dt);
-      sc_lds[threadIdx.x * 4 + 1] = dt;
-    }
-    if (KIND == kScanLogGates && rp == 0) {
-      const float li = p.cap * tanhf((areg + gate_a) / p.cap);
-      const float lf = log_sigmoidf_(p.cap * tanhf((breg + gate_b) / p.cap));
-      float before = 0.0f, after = 0.0f;           // the running maximum on either side of this lane's token
-      for (int i = 0; i < cn; ++i) {
-        const float fi = __shfl(lf, i, kWave), ii = __shfl(li, i, kWave);
-        const float nm = fmaxf(fi + m, ii);
-        if (lane == i) {
-          before = m;
-          after = nm;
-        }
-        m = nm;
-      }
-      if (lane < CH) {
-        sc_lds[lane * 4] = expf(lf + before - after);
-        sc_lds[lane * 4 + 1] = expf(li - after);
-        sc_lds[lane * 4 + 2] = expf(-after);
-      }
-    }
     __syncthreads();
     if (c0 + CH < n) fetch(c0 + CH);
     for (int i = 0; i < cn; ++i) {
-      float vv = v_lds[i * kWave + lane];
-      float dec = 1.0f;
+      float4 vv = *reinterpret_cast<const float4*>(v_lds + i * kWave + (lane & ~3));
       if (KIND != kScanRowDecay) {
-        const float2 dw = *reinterpret_cast<const float2*>(sc_lds + i * 4);
-        dec = dw.x;
-        if (KIND == kScanLogGates && owner) {
-          const int at = i * DP + row0 + (lane < DR ? lane : 0);
-          nstate = dec * nstate + dw.y * k_lds[at];
-          const float share = row16_sum(lane < DR ? nstate * q_lds[at] : 0.0f);
-          if (lane < DR && (lane & 15) == 0) x_lds[(i * NW + rp) * R16 + (lane >> 4)] = share;
-        }
-        vv *= dw.y;
-      }
-      float po4[4] = {0.0f, 0.0f, 0.0f, 0.0f};     // four chains: one sum would be bound by its own latency
+        const float2 mw = *reinterpret_cast<const float2*>(sc_lds + i * 4);
+        if (__builtin_amdgcn_readfirstlane(__builtin_bit_cast(int, mw.x)) != __builtin_bit_cast(int, 1.0f)) {
 #pragma unroll
-      for (int r = 0; r < DR; r += 4) {
-        const float4 k4 = *reinterpret_cast<const float4*>(k_lds + i * DP + row0 + r);
-        const float4 q4 = *reinterpret_cast<const float4*>(q_lds + i * DP + row0 + r);
-        if (KIND == kScanRowDecay) {               // read before this token decays and writes
-          const float4 w4 = *reinterpret_cast<const float4*>(x_lds + i * DP + row0 + r);
-          po4[0] += s[r] * q4.x;
-          po4[1] += s[r + 1] * q4.y;
-          po4[2] += s[r + 2] * q4.z;
-          po4[3] += s[r + 3] * q4.w;
-          s[r] = w4.x * s[r] + k4.x * vv;
-          s[r + 1] = w4.y * s[r + 1] + k4.y * vv;
-          s[r + 2] = w4.z * s[r + 2] + k4.z * vv;
-          s[r + 3] = w4.w * s[r + 3] + k4.w * vv;
-        } else {
-          s[r] = dec * s[r] + k4.x * vv;
-          s[r + 1] = dec * s[r + 1] + k4.y * vv;
-          s[r + 2] = dec * s[r + 2] + k4.z * vv;
-          s[r + 3] = dec * s[r + 3] + k4.w * vv;
-          po4[0] += s[r] * q4.x;
-          po4[1] += s[r + 1] * q4.y;
-          po4[2] += s[r + 2] * q4.z;
-          po4[3] += s[r + 3] * q4.w;
+          for (int r = 0; r < RL; ++r)
+#pragma unroll
+            for (int c = 0; c < 4; ++c) s[r][c] *= mw.x;
+        }
+        vv.x *= mw.y; vv.y *= mw.y; vv.z *= mw.y; vv.w *= mw.y;
+      }
+      float kr[RL], qr[RL], wr[KIND == kScanRowDecay ? RL : 1];
+      lds_rows<RL>(k_lds + i * DP + own0, kr);
+      lds_rows<RL>(q_lds + i * DP + own0, qr);
+      if constexpr (KIND == kScanRowDecay) lds_rows<RL>(x_lds + i * DP + own0, wr);
+      const float v4[4] = {vv.x, vv.y, vv.z, vv.w};
+      float po[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+#pragma unroll
+      for (int r = 0; r < RL; ++r) {
+#pragma unroll
+        for (int c = 0; c < 4; ++c) {
+          if constexpr (KIND == kScanRowDecay) {   // read before this token decays and writes
+            po[c] += s[r][c] * qr[r];
+            s[r][c] = wr[r] * s[r][c] + kr[r] * v4[c];
+          } else {
+            s[r][c] += kr[r] * v4[c];
+            po[c] += s[r][c] * qr[r];
+          }
         }
       }
-      part_o[(i * NW + rp) * kWave + lane] = (po4[0] + po4[1]) + (po4[2] + po4[3]);
+      part_o[(i * NW + rp) * kWave + lane] = quad_columns(po, rl);
     }
+    if (owner && nr >= 0)
+      for (int i = 0; i < cn; ++i) {
+        const float2 mw = *reinterpret_cast<const float2*>(sc_lds + i * 4);
+        nstate = nstate * mw.x + mw.y * k_lds[i * DP + nr];
+        const float share = row16_sum(nstate * q_lds[i * DP + nr]);
+        if ((lane & 15) == 0) x_lds[i * (DP / 16) + nr / 16] = share;
+      }
+    if (KIND != kScanRowDecay && rp == 0 && c0 + CH < n) scalars(min(CH, n - c0 - CH), sc_all + (buf ^ 1) * 4 * CH);
     __syncthreads();
     for (int x = threadIdx.x; x < cn * kWave; x += NT) {
       const int tok = x / kWave, ln = x % kWave, cc = blockIdx.x * kWave + ln;
@@ -495,6 +573,7 @@ __global__ __launch_bounds__(NW * 64, DR > 32 ? 2 : (KIND == kScanRowDecay && DR
       float sum = 0.0f;
 #pragma unroll
       for (int w = 0; w < NW; w += 2) sum += po[w * kWave] + po[(w + 1) * kWave];
+      if (KIND != kScanRowDecay) sum *= sc_lds[tok * 4 + 2];
       if (KIND == kScanStep) sum += skip * v_lds[x];
       if (KIND == kScanRowDecay) {
         float bon = bon_lds[tok * SEG];
@@ -504,25 +583,29 @@ __global__ __launch_bounds__(NW * 64, DR > 32 ? 2 : (KIND == kScanRowDecay && DR
       }
       if (cc < p.Dv) p.o[((static_cast<int64_t>(q0) + c0 + tok) * p.H + h) * p.Dv + cc] = sum;
     }
-    if (owner) {                                   // |n . q| of the chunk's tokens, NT / CH threads each
-      constexpr int PER = NT / CH < kWave ? NT / CH : kWave;
-      const int tok = threadIdx.x / PER, part = threadIdx.x % PER;
+    if (owner && threadIdx.x < cn) {
+      const float* sh = x_lds + threadIdx.x * (DP / 16);
       float nq = 0.0f;
-      if (tok < cn)
-        for (int d = part; d < NW * R16; d += PER) nq += x_lds[tok * NW * R16 + d];
-#pragma unroll
-      for (int off = PER / 2; off > 0; off >>= 1) nq += __shfl_xor(nq, off, kWave);
-      if (tok < cn && part == 0)
-        p.den[(static_cast<int64_t>(q0) + c0 + tok) * p.H + h] = fmaxf(fabsf(nq), sc_lds[tok * 4 + 2]) + 1e-6f;
+      for (int e = 0; e < DP / 16; ++e) nq += sh[e];
+      p.den[(static_cast<int64_t>(q0) + c0 + threadIdx.x) * p.H + h] =
+          fmaxf(fabsf(nq) * sc_lds[threadIdx.x * 4 + 2], sc_lds[threadIdx.x * 4 + 3]) + 1e-6f;
     }
+    if (KIND != kScanRowDecay && c0 + CH >= n) last_factor = sc_lds[(cn - 1) * 4 + 2];
     __syncthreads();                               // the next chunk overwrites the values and scalars read above
   }
-  if (live) {
 #pragma unroll
-    for (int r = 0; r < DR; ++r)
-      if (row0 + r < p.D) sbase[static_cast<int64_t>(row0 + r) * p.Dv + col] = s[r];
+  for (int r = 0; r < RL; ++r) {
+    float* dst = sbase + static_cast<int64_t>(own0 + r) * p.Dv + col0;
+    if (own0 + r >= p.D) continue;
+    if (whole) {
+      st4(dst, float4{s[r][0] * last_factor, s[r][1] * last_factor, s[r][2] * last_factor, s[r][3] * last_factor});
+    } else {
+#pragma unroll
+      for (int c = 0; c < 4; ++c)
+        if (col0 + c < p.Dv) dst[c] = s[r][c] * last_factor;
+    }
   }
-  if (nrow) p.norm_state[head * p.D + row0 + lane] = nstate;
+  if (nrow) p.norm_state[head * p.D + nr] = nstate * last_factor;
   if (KIND == kScanLogGates && threadIdx.x == 0) *mplace = m;
 }
 

@@ -44,7 +44,7 @@ class MatrixMemory(nn.Module):
     # -- cache protocol of the model runner
     @property
     def _copies(self) -> int:
-        return -(-self.Dv // mix_ops.SCAN_COLUMNS)      # of the running maximum: one per workgroup of a head
+        return mix_ops.scan_copies(self.Dv)
 
     def cache_bytes(self, block_size: int, act_bytes: int) -> tuple[int, int]:
         """(bytes per cache page, bytes per state slot)."""

@@ -1121,7 +1121,12 @@ def token_shift(h, mu, state, step):
 
 
 SCAN_STEP, SCAN_LOG_GATES, SCAN_ROW_DECAY = 0, 1, 2
-SCAN_COLUMNS = 64          # value columns of one workgroup of the scan (one copy of the running maximum each)
+SCAN_COLUMNS = 64          # value columns of one workgroup of the scan
+
+
+def scan_copies(Dv: int) -> int:
+    """Copies of the running maximum that SCAN_LOG_GATES keeps: one per workgroup of a head."""
+    return -(-Dv // SCAN_COLUMNS)
 
 
 def gated_scan(kind, q, k, v, a, p0, p1, step, state, H, G, D, Dv, a2=None, p2=None, q_scale=1.0, cap=1.0, norm_state=None,
@@ -1133,7 +1138,7 @@ def gated_scan(kind, q, k, v, a, p0, p1, step, state, H, G, D, Dv, a2=None, p2=N
                       write = dt, o += p2 v
       SCAN_LOG_GATES  a, a2 act [T, H], p0, p1 their biases (f32 [H]): i = cap tanh((a + p0)/cap), f = logsigmoid(cap
                       tanh((a2 + p1)/cap)), m' = max(f + m, i) with m from 0; decay = e^(f+m-m'), write = e^(i-m');
-                      n <- decay n + write k beside S. norm_state f32 [slots, H, D], max_state f32 [slots, H, ceil(Dv/64)]
+                      n <- decay n + write k beside S. norm_state f32 [slots, H, D], max_state f32 [slots, H, scan_copies(Dv)]
       SCAN_ROW_DECAY  a act [T, H*D], p0, p1 f32 [H*D]: w = exp(-exp(a + p0)) for each row of S; o = (S + diag(p1) k v^T)^T q
                       before S <- diag(w) S + k v^T
     q is multiplied by q_scale (not in SCAN_ROW_DECAY). Returns o f32 [T, H, Dv], and for SCAN_LOG_GATES also
@@ -1145,7 +1150,7 @@ def gated_scan(kind, q, k, v, a, p0, p1, step, state, H, G, D, Dv, a2=None, p2=N
     o = torch.empty(T, H, Dv, dtype=torch.float32, device=q.device)
     den = None
     if kind == SCAN_LOG_GATES:
-        assert norm_state.shape[1:] == (H, D) and max_state.shape[1:] == (H, -(-Dv // SCAN_COLUMNS)) and a2.stride(0) == a.stride(0)
+        assert norm_state.shape[1:] == (H, D) and max_state.shape[1:] == (H, scan_copies(Dv)) and a2.stride(0) == a.stride(0)
         den = torch.empty(T, H, dtype=torch.float32, device=q.device)
     if q.is_cuda:
         assert all(x.stride(1) == 1 for x in (q, k, v, a))

@@ -271,7 +271,7 @@ def case_scan_log_gates(device, dtype):
                 want[i, h] = oracle.unit_rms(o, 1e-5) * nw[h * Dv:(h + 1) * Dv].to(F64) * torch.sigmoid(gate[i][:, h * Dv:(h + 1) * Dv].to(F64))
         state = torch.full((3, H, D, Dv), 7.0, device=device)
         ns = torch.full((3, H, D), 3.0, device=device)
-        ms = torch.full((3, H, -(-Dv // 64)), 11.0, device=device)
+        ms = torch.full((3, H, mix_ops.scan_copies(Dv)), 11.0, device=device)
         bid, bfd, nwd = bi.to(device), bf.to(device), nw.to(device)
 
         def run(parts):
