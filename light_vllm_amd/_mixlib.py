@@ -1,6 +1,6 @@
 """ctypes binding of liblvmix.so (include/lv_mixers.h): the kernels of the recurrent and windowed
-sequence mixers (delta rule, windowed and latent attention), the residual streams, the gated units
-and the mixture-of-experts router.
+sequence mixers (delta rule, gated scans, windowed and latent attention), the residual streams, the
+gated units and the mixture-of-experts router.
 
 The library is separate from liblvattn.so so that a model that needs only these kernels builds
 only these: `load()` compiles the sources once when no built library is there (a fresh checkout),

@@ -11,6 +11,7 @@
 //                             and what is written are computed in f32 as the inputs are staged, from one of three rules:
 //                             step sizes of a state-space layer, log gates under a running maximum with a normaliser
 //                             vector beside the state, or a decay per row of the state with a bonus for the current token.
+//                             A lane owns a block of rows by four columns of the state.
 //   grouped_gate_norm_kernel  o silu(z), RMS norm in equal parts of the row, weight.
 //   residual_pair_norm_kernel the f32 residual receives the scaled sum of two RMS-normed and weighted sublayer outputs and
 //                             is normed for the next sublayer.
