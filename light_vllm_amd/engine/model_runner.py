@@ -319,7 +319,7 @@ class ModelRunner:
         clamp instead of faulting, so the range is enforced here, where the lengths are known."""
         limit = getattr(self, "max_position", None)     # None: a bare runner built for its step-input builders
         if limit is not None and last_position >= limit:
-            raise IndexError(f"position {last_position} is outside the position table of {limit} rows "
+            raise IndexError(f"position {last_position} is outside the rotary table or position table of {limit} rows "
                              "(sequence longer than max_position_embeddings)")
 
     def _to_device(self, values, dtype) -> torch.Tensor:
