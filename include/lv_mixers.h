@@ -59,6 +59,12 @@
  *   lv_residual_pair_norm    single f32 residual: adds the scaled sum of two RMS-normed and weighted sublayer outputs, RMS norm
  *   lv_embed_norm            scaled token row + hashed pair row + position row, RMS norm, the first sublayer's RMS norm
  *   lv_unary_act             activation without a gate
+ *   lv_latent_store          lv_latent_prep and lv_latent_q_finish in one for queries that come straight from the input, with the
+ *                            pairing of rotated entries and a factor on cosines and sines as choices
+ *   lv_head_norm_store       per-head RMS norm of the queries, keys stored as they are with the factor of their norm beside them
+ *   lv_gated_linear_recurrence   Griffin's RG-LRU: block-diagonal gates, S <- a S + sqrt(1 - a^2) i u per channel, gelu branch
+ *   lv_scaled_embedding      token rows times a constant as the f32 residual
+ *   lv_residual_split        residual update, and the residual as the sum of two bf16 numbers for a matrix product
  *
  * A "ragged step" is a batch of B sequences; sequence b brings cu_q[b+1]-cu_q[b] new tokens that
  * follow ctx_lens[b] tokens already in the cache / state (a whole prompt, a portion of one, or one
@@ -80,7 +86,7 @@
 extern "C" {
 #endif
 
-#define LV_MIX_ABI_VERSION 8
+#define LV_MIX_ABI_VERSION 9
 #define LV_MIX_BF16 0
 #define LV_MIX_F32 1
 #define LV_MIX_MAX_STREAMS 8
@@ -92,6 +98,8 @@ extern "C" {
 #define LV_MIX_ACT_GELU_ERF 1     /* z Phi(z), exact */
 #define LV_MIX_ACT_GELU_TANH 2    /* 0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3))) */
 #define LV_MIX_ACT_TANH 3
+#define LV_MIX_ACT_RELU 4         /* max(z, 0) */
+#define LV_MIX_ACT_MAX 4
 #define LV_MIX_SCAN_STEP 0        /* lv_gated_scan: how a state decays and what it takes, see there */
 #define LV_MIX_SCAN_LOG_GATES 1
 #define LV_MIX_SCAN_ROW_DECAY 2
@@ -300,17 +308,28 @@ int lv_qk_prep_store(const void* proj, int64_t ld, int off_q, int off_k, int off
  * (kept first tokens and chunks do not combine with pooled blocks, P > 0). sinks f32 [H] (may be NULL): the denominator of
  * head h's softmax also holds exp(sinks[h]); has_sink without sinks: exp(0). softcap > 0: the score q.k * scale becomes
  * softcap * tanh(score / softcap). */
+/* What lv_masked_attn(_mfma) can be given beyond that (a NULL pointer: none of it).
+ * key_scale f32 [pages, page, G] or NULL: the score of a cached key is multiplied by its number as well (keys kept unnormed).
+ * dist_bias f32 [H, bias_len] or NULL: head h's score at distance n = i - j gets dist_bias[h, min(n, bias_len - 1)] added, after all
+ * factors. These two combine with windows, kept tokens, chunks and sinks. out_ld: elements between two tokens' output rows (0: H*Dv). */
+typedef struct lv_attn_extras {
+  const void* key_scale;
+  const void* dist_bias;
+  int32_t bias_len;
+  int64_t out_ld;
+} lv_attn_extras;
 int lv_masked_attn(const void* q, const void* k_cache, const void* v_cache, const void* kp, const void* vp,
                    const void* gate, int64_t ld_gate, void* out, const int32_t* cu_q, const int32_t* ctx_lens,
                    const int32_t* tok_seq, const int32_t* block_tables, int bt_stride, int64_t T, int H, int G, int D,
                    int Dv, int page, int window, int keep_first, int chunk, int P, float scale, float softcap, int has_sink,
-                   const void* sinks, int64_t k_ld, int64_t v_ld, int gate_kind, int dtype, void* stream);
+                   const void* sinks, int64_t k_ld, int64_t v_ld, int gate_kind, const lv_attn_extras* extras, int dtype,
+                   void* stream);
 int lv_masked_attn_mfma(const void* q, const void* k_cache, const void* v_cache, const void* kp, const void* vp,
                         const void* gate, int64_t ld_gate, void* out, const int32_t* cu_q, const int32_t* ctx_lens,
                         const int32_t* block_tables, int bt_stride, int B, int max_new_tokens, int H, int G, int D,
                         int Dv, int page, int window, int keep_first, int chunk, int P, float scale, float softcap, int has_sink,
                         const void* sinks, int nsplit, void* workspace, int64_t T, int64_t k_ld, int64_t v_ld,
-                        int gate_kind, void* stream);
+                        int gate_kind, const lv_attn_extras* extras, void* stream);
 
 /* proj act [T, ld]: H query heads of D at column off_q, H key heads of D at off_k, H value heads of Dv at off_v; each entry
  * passes silu first. Per head and token: S <- decay[h] * S + k v^T; o = S^T q. state f32 [slots, H, D, Dv], read unless
@@ -319,8 +338,8 @@ int lv_lightning_attn(const void* proj, int64_t ld, int off_q, int off_k, int of
                       const int32_t* cu_q, const int32_t* ctx_lens, const int32_t* slots, void* o, int B, int H, int D, int Dv,
                       int dtype, void* stream);
 
-/* in act [T, 2F] (row stride ld_in) = [gate | up];  out act [T, F] = act(gate) * up, act one of LV_MIX_ACT_*. */
-int lv_glu_act(const void* in, int64_t ld_in, void* out, int64_t T, int F, int act, int dtype, void* stream);
+/* in act [T, 2F] (row stride ld_in) = [gate | up];  out act [T, F] (row stride ld_out) = act(gate) * up, act one of LV_MIX_ACT_*. */
+int lv_glu_act(const void* in, int64_t ld_in, void* out, int64_t ld_out, int64_t T, int F, int act, int dtype, void* stream);
 
 /* lv_moe_route with the scores as sigmoid or as softmax over all E logits of the row (LV_MIX_SCORE_*), and the rank of a
  * group as the sum of its two highest selection scores or its highest (LV_MIX_GROUP_*). */
@@ -409,6 +428,43 @@ int lv_embed_norm(const void* ids, const void* table, int vocab, float scale, co
 
 /* out act [n] = act(in), act one of LV_MIX_ACT_*. */
 int lv_unary_act(const void* in, void* out, int64_t n, int act, int dtype, void* stream);
+
+/* Latent attention whose queries come straight from the input. proj act [T, ld]: H queries of Dn + Dr at column off_q (rotated
+ * part last), the latent at off_kv (R wide) followed by the positional key part (Dr wide).  cache act [pages, page, R + Dr]: the
+ * token's row receives rms_norm(latent) * kv_w | rotated positional part;  q_out act [T, H, R + Dr]: entries R .. R + Dr - 1 of every
+ * head receive the rotated query part (the others are left alone).  Of the first rot_dims (even, <= Dr) entries, 2i pairs with 2i + 1
+ * (interleaved) or i with i + rot_dims/2; angle = position * inv_freq[i], cosines and sines times `magnitude`. */
+int lv_latent_store(const void* proj, int64_t ld, int off_q, int off_kv, const void* kv_w, const void* inv_freq, float magnitude,
+                    void* q_out, void* cache, const int32_t* cu_q, const int32_t* ctx_lens, const int32_t* tok_seq,
+                    const int32_t* block_tables, int bt_stride, int64_t T, int H, int Dn, int Dr, int R, int rot_dims, int interleaved,
+                    int page, float eps, int dtype, void* stream);
+
+/* proj act [T, ld]: H query heads of D at column off_q, G key heads of D at off_k.  q_out act [T, H*D] = head / sqrt(mean(head^2) +
+ * eps) * q_w (f32 [D]); keys into cache act [pages, page, G, D] as they are, 1 / sqrt(mean(head^2) + eps) into key_scale f32
+ * [pages, page, G]. */
+int lv_head_norm_store(const void* proj, int64_t ld, int off_q, int off_k, const void* q_w, void* q_out, void* cache, void* key_scale,
+                       const int32_t* cu_q, const int32_t* ctx_lens, const int32_t* tok_seq, const int32_t* block_tables, int bt_stride,
+                       int64_t T, int H, int G, int D, int page, float eps, int dtype, void* stream);
+
+/* Real-gated linear recurrent unit over the new tokens of every sequence, channel by channel. u, y act [T, N] (row strides ldu,
+ * ldy); the N channels are `blocks` parts of n = N / blocks; gate_w act [blocks, 2, n, n] ([out, in]), gate_b f32 [blocks, 2, n],
+ * rate f32 [N]:  r, i = sigmoid(gate_w[b, 0|1] u_b + gate_b[b, 0|1]);  log a = rate r;  S <- a S + sqrt(1 - a^2) i u;
+ * out act [T, N] (row stride ldo) = S gelu_tanh(y).  state f32 [slots, N], taken as zero for a sequence with no context, written back.
+ * mfma != 0 (bf16, n a multiple of 32, u rows 16-byte aligned): the gates on the matrix cores, 64 tokens a tile; nsplit > 1: a
+ * sequence's tiles are cut into nsplit parts, which need workspace f32 [B, nsplit, 2, N]. max_new_tokens = the largest
+ * cu_q[b+1] - cu_q[b]; steps of single tokens take a kernel of their own. */
+int lv_gated_linear_recurrence(const void* u, int64_t ldu, const void* y, int64_t ldy, const void* gate_w, const void* gate_b,
+                               const void* rate, void* state, const int32_t* cu_q, const int32_t* ctx_lens, const int32_t* slots,
+                               void* out, int64_t ldo, int B, int64_t T, int max_new_tokens, int N, int blocks, int nsplit,
+                               void* workspace, int mfma, int dtype, void* stream);
+
+/* ids int64 [T], table act [vocab, W]:  x f32 [T, W] = table[id] * scale;  rows act [T, W] (NULL: none) = table[id];  split bf16
+ * [T, 2W] (NULL: none) = x as lv_residual_split leaves it. */
+int lv_scaled_embedding(const void* ids, const void* table, int vocab, float scale, void* x, void* rows, void* split, int64_t T, int W,
+                        int dtype, void* stream);
+
+/* x f32 [T, W] += y (bf16 [T, W], may be NULL);  out bf16 [T, 2W] = x rounded | (x - x rounded) rounded. */
+int lv_residual_split(void* x, const void* y, void* out, int64_t T, int W, void* stream);
 
 #ifdef __cplusplus
 }

@@ -1,5 +1,5 @@
 """ctypes binding of liblvmix.so (include/lv_mixers.h): the kernels of the recurrent and windowed
-sequence mixers (delta rule, gated scans, windowed and latent attention), the residual streams, the
+sequence mixers (delta rule, gated scans, gated linear recurrence, windowed and latent attention), the residual streams, the
 gated units and the mixture-of-experts router.
 
 The library is separate from liblvattn.so so that a model that needs only these kernels builds
@@ -17,8 +17,8 @@ _HERE = os.path.dirname(os.path.abspath(__file__))
 CSRC = os.path.join(_HERE, "csrc", "mixers")
 LIB_PATH = os.path.join(_HERE, "lib", "liblvmix.so")
 SOURCES = ["mix_stream.hip", "mix_window_attn.hip", "mix_window_mfma.hip", "mix_latent.hip", "mix_moe_gemm.hip",
-           "mix_sandwich.hip", "mix_parallel.hip", "mix_recurrent.hip"]
-ABI_VERSION = 8
+           "mix_sandwich.hip", "mix_parallel.hip", "mix_recurrent.hip", "mix_prep.hip", "mix_lru.hip"]
+ABI_VERSION = 9
 
 _P = c_void_p
 SIGNATURES = {
@@ -63,12 +63,12 @@ SIGNATURES = {
     "lv_qk_prep_store": (c_int, [_P, c_int64, c_int, c_int, c_int, _P, _P, _P, _P, _P, _P, _P, _P, _P, c_int, c_int64,
                                  c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int, _P]),
     "lv_masked_attn": (c_int, [_P, _P, _P, _P, _P, _P, c_int64, _P, _P, _P, _P, _P, c_int, c_int64, c_int, c_int, c_int, c_int,
-                               c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_int, _P, c_int64, c_int64, c_int, c_int, _P]),
+                               c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_int, _P, c_int64, c_int64, c_int, _P, c_int, _P]),
     "lv_masked_attn_mfma": (c_int, [_P, _P, _P, _P, _P, _P, c_int64, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, c_int,
                                     c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_int, _P, c_int, _P, c_int64, c_int64,
-                                    c_int64, c_int, _P]),
+                                    c_int64, c_int, _P, _P]),
     "lv_lightning_attn": (c_int, [_P, c_int64, c_int, c_int, c_int, _P, _P, _P, _P, _P, _P, c_int, c_int, c_int, c_int, c_int, _P]),
-    "lv_glu_act": (c_int, [_P, c_int64, _P, c_int64, c_int, c_int, c_int, _P]),
+    "lv_glu_act": (c_int, [_P, c_int64, _P, c_int64, c_int64, c_int, c_int, c_int, _P]),
     "lv_moe_route_scored": (c_int, [_P, _P, _P, _P, _P, c_int64, c_int, c_int, c_int, c_int, c_int, c_int, c_int, _P]),
     "lv_expert_act_scale": (c_int, [_P, _P, c_int64, _P, c_int64, c_int, c_int, c_int, c_int, _P]),
     "lv_moe_grouped_act_ff": (c_int, [_P, _P, _P, _P, _P, _P, _P, c_int64, c_int, c_int, c_int, c_int, c_int, c_int, _P]),
@@ -86,7 +86,20 @@ SIGNATURES = {
     "lv_embed_norm": (c_int, [_P, _P, c_int, c_float, _P, c_int, c_int64, c_int64, _P, _P, c_int, _P, _P, c_float, c_float, _P, _P,
                               _P, _P, _P, _P, c_int64, c_int, c_int, _P]),
     "lv_unary_act": (c_int, [_P, _P, c_int64, c_int, c_int, _P]),
+    "lv_latent_store": (c_int, [_P, c_int64, c_int, c_int, _P, _P, c_float, _P, _P, _P, _P, _P, _P, c_int, c_int64, c_int, c_int, c_int,
+                                c_int, c_int, c_int, c_int, c_float, c_int, _P]),
+    "lv_head_norm_store": (c_int, [_P, c_int64, c_int, c_int, _P, _P, _P, _P, _P, _P, _P, _P, c_int, c_int64, c_int, c_int, c_int, c_int,
+                                   c_float, c_int, _P]),
+    "lv_gated_linear_recurrence": (c_int, [_P, c_int64, _P, c_int64, _P, _P, _P, _P, _P, _P, _P, _P, c_int64, c_int, c_int64, c_int,
+                                           c_int, c_int, c_int, _P, c_int, c_int, _P]),
+    "lv_scaled_embedding": (c_int, [_P, _P, c_int, c_float, _P, _P, _P, c_int64, c_int, c_int, _P]),
+    "lv_residual_split": (c_int, [_P, _P, _P, c_int64, c_int, _P]),
 }
+
+class AttnExtras(ctypes.Structure):
+    """lv_attn_extras of the header."""
+    _fields_ = [("key_scale", c_void_p), ("dist_bias", c_void_p), ("bias_len", ctypes.c_int32), ("out_ld", c_int64)]
+
 
 _lib = None
 

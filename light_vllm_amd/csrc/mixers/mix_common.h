@@ -80,7 +80,7 @@ __device__ __forceinline__ float mix_act(float v, int act) {
   if (act == LV_MIX_ACT_GELU_TANH) return gelu_tanh_(v);
   if (act == LV_MIX_ACT_TANH) return tanhf(v);
   v = fmaxf(v, 0.0f);
-  return v * v;
+  return act == LV_MIX_ACT_RELU ? v : v * v;
 }
 
 int fail(int code, const char* fmt, ...);

@@ -363,8 +363,8 @@ static int lightning_dispatch(const LightningParams& p, int B, hipStream_t s) {
 
 // ------------------------------------------------------------------------------------------------
 template <typename T, int VEC>
-__global__ __launch_bounds__(256) void glu_act_kernel(const T* __restrict__ in, int64_t ld_in, T* __restrict__ out, int64_t Tn,
-                                                      int F, int act) {
+__global__ __launch_bounds__(256) void glu_act_kernel(const T* __restrict__ in, int64_t ld_in, T* __restrict__ out, int64_t ld_out,
+                                                      int64_t Tn, int F, int act) {
   const int64_t idx = (static_cast<int64_t>(blockIdx.x) * blockDim.x + threadIdx.x) * VEC;
   if (idx >= Tn * F) return;
   const int64_t t = idx / F;
@@ -372,10 +372,10 @@ __global__ __launch_bounds__(256) void glu_act_kernel(const T* __restrict__ in, 
   const T* row = in + t * ld_in;
   if constexpr (VEC == 4) {
     const float4 g = ld4(row + f), u = ld4(row + F + f);
-    st4(out + idx, float4{mix_act(g.x, act) * u.x, mix_act(g.y, act) * u.y, mix_act(g.z, act) * u.z,
+    st4(out + t * ld_out + f, float4{mix_act(g.x, act) * u.x, mix_act(g.y, act) * u.y, mix_act(g.z, act) * u.z,
                           mix_act(g.w, act) * u.w});
   } else {
-    stf(out + idx, mix_act(ldf(row + f), act) * ldf(row + F + f));
+    stf(out + t * ld_out + f, mix_act(ldf(row + f), act) * ldf(row + F + f));
   }
 }
 
@@ -491,16 +491,16 @@ int lv_lightning_attn(const void* proj, int64_t ld, int off_q, int off_k, int of
   return launched("lv_lightning_attn");
 }
 
-int lv_glu_act(const void* in, int64_t ld_in, void* out, int64_t T, int F, int act, int dtype, void* stream) {
+int lv_glu_act(const void* in, int64_t ld_in, void* out, int64_t ld_out, int64_t T, int F, int act, int dtype, void* stream) {
   if (T == 0) return 0;
-  if (!in || !out || T < 0 || F <= 0 || ld_in < 2 * static_cast<int64_t>(F) || act < 0 || act > LV_MIX_ACT_GELU_TANH)
+  if (!in || !out || T < 0 || F <= 0 || ld_in < 2 * static_cast<int64_t>(F) || ld_out < F || act < 0 || act > LV_MIX_ACT_MAX)
     return fail(-1, "lv_glu_act: bad arguments");
-  const bool vec4 = F % 4 == 0 && ld_in % 4 == 0 && (reinterpret_cast<uintptr_t>(in) & 15) == 0 &&
+  const bool vec4 = F % 4 == 0 && ld_in % 4 == 0 && ld_out % 4 == 0 && (reinterpret_cast<uintptr_t>(in) & 15) == 0 &&
                     (reinterpret_cast<uintptr_t>(out) & 15) == 0;
   const int64_t n = T * F / (vec4 ? 4 : 1);
   dim3 grid(static_cast<unsigned>((n + 255) / 256)), block(256);
 #define LVMIX_GLU(TT, VV)                                                                                                  \
-  glu_act_kernel<TT, VV><<<grid, block, 0, as_stream(stream)>>>(static_cast<const TT*>(in), ld_in, static_cast<TT*>(out), T, F, act)
+  glu_act_kernel<TT, VV><<<grid, block, 0, as_stream(stream)>>>(static_cast<const TT*>(in), ld_in, static_cast<TT*>(out), ld_out, T, F, act)
   if (dtype == LV_MIX_BF16) {
     if (vec4) LVMIX_GLU(bf16_t, 4); else LVMIX_GLU(bf16_t, 1);
   } else if (dtype == LV_MIX_F32) {

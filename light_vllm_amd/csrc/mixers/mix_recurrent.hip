@@ -1083,7 +1083,7 @@ int lv_embed_norm(const void* ids, const void* table, int vocab, float scale, co
 
 int lv_unary_act(const void* in, void* out, int64_t n, int act, int dtype, void* stream) {
   if (n == 0) return 0;
-  if (!in || !out || n < 0 || act < 0 || act > LV_MIX_ACT_TANH) return fail(-1, "lv_unary_act: bad arguments");
+  if (!in || !out || n < 0 || act < 0 || act > LV_MIX_ACT_MAX) return fail(-1, "lv_unary_act: bad arguments");
   const bool vec4 = n % 4 == 0 && aligned16(in) && aligned16(out);
   dim3 grid(static_cast<unsigned>((n / (vec4 ? 4 : 1) + 255) / 256)), block(256);
   if (dtype == LV_MIX_BF16) {

@@ -90,6 +90,10 @@ struct WindowAttnParams {
   int chunk;            // > 0: a query sees its own chunk of that many positions (counted from 0) up to itself; no window
   const float* sinks;   // [H] or NULL: a learned score per query head in place of the sink's 0
   float softcap;        // > 0: scores pass softcap * tanh(score / softcap)
+  const float* key_scale;   // [pages, page, G] or NULL: a factor on the score of every cached key
+  const float* dist_bias;   // [H, bias_len] or NULL: added to the score at distance min(pos - key, bias_len - 1)
+  int bias_len;
+  int64_t out_ld;       // elements between the output rows of two tokens
 };
 
 // kMaxRep: query heads of one kv head served by one workgroup; kMaxDvi: value columns per lane (Dv <= 64 * kMaxDvi).
@@ -142,13 +146,18 @@ __global__ __launch_bounds__(256) void window_pool_attn_kernel(WindowAttnParams 
     const bool valid = idx < nkeys;
     // row of this lane's key in its cache
     const T* krow = kc;
+    float kfactor = 1.0f;
+    int dist = 0;
     if (valid) {
       if (idx < nb) {
         const int pj = (idx * p.P + p.P - 1) / p.page;
         krow = kpool + (static_cast<int64_t>(bt[pj]) * p.PP + (idx - (p.page * pj) / p.P)) * GD + g * D;
       } else {
         const int j = idx < nb + nf ? idx - nb : j0 + idx - nb - nf;
-        krow = kc + (static_cast<int64_t>(bt[j / p.page]) * p.page + j % p.page) * p.k_ld + g * D;
+        const int64_t slot = static_cast<int64_t>(bt[j / p.page]) * p.page + j % p.page;
+        krow = kc + slot * p.k_ld + g * D;
+        if (p.key_scale != nullptr) kfactor = p.key_scale[slot * p.G + g];
+        dist = min(pos - j, p.bias_len - 1);
       }
     }
     float s[kMaxRep];
@@ -165,6 +174,8 @@ __global__ __launch_bounds__(256) void window_pool_attn_kernel(WindowAttnParams 
 #pragma unroll
     for (int h = 0; h < kMaxRep; ++h) {
       if (h < rep) {
+        if (p.key_scale != nullptr) s[h] *= kfactor;
+        if (p.dist_bias != nullptr && valid) s[h] += p.dist_bias[static_cast<int64_t>(h0 + h) * p.bias_len + dist];
         if (p.softcap > 0.0f) s[h] = p.softcap * tanhf(s[h] / p.softcap);
         const float cm = wave_max(valid ? s[h] : -INFINITY);
         const float nm = fmaxf(m[h], cm);
@@ -217,7 +228,7 @@ __global__ __launch_bounds__(256) void window_pool_attn_kernel(WindowAttnParams 
     }
   }
   __syncthreads();
-  T* out = static_cast<T*>(p.out) + t * p.H * Dv;
+  T* out = static_cast<T*>(p.out) + t * p.out_ld;
   const T* gate = p.gate != nullptr ? static_cast<const T*>(p.gate) + t * p.ld_gate : nullptr;
   for (int i = threadIdx.x; i < rep * Dv; i += blockDim.x) {
     const int h = i / Dv, dv = i - h * Dv;
@@ -296,14 +307,15 @@ int lv_window_pool_attn(const void* q, const void* k_cache, const void* v_cache,
                         int Dv, int page, int window, int P, float scale, int has_sink, int64_t k_ld, int64_t v_ld,
                         int gate_kind, int dtype, void* stream) {
   return lv_masked_attn(q, k_cache, v_cache, kp, vp, gate, ld_gate, out, cu_q, ctx_lens, tok_seq, block_tables, bt_stride, T, H,
-                        G, D, Dv, page, window, 0, 0, P, scale, 0.0f, has_sink, nullptr, k_ld, v_ld, gate_kind, dtype, stream);
+                        G, D, Dv, page, window, 0, 0, P, scale, 0.0f, has_sink, nullptr, k_ld, v_ld, gate_kind, nullptr, dtype, stream);
 }
 
 int lv_masked_attn(const void* q, const void* k_cache, const void* v_cache, const void* kp, const void* vp,
                    const void* gate, int64_t ld_gate, void* out, const int32_t* cu_q, const int32_t* ctx_lens,
                    const int32_t* tok_seq, const int32_t* block_tables, int bt_stride, int64_t T, int H, int G, int D,
                    int Dv, int page, int window, int keep_first, int chunk, int P, float scale, float softcap, int has_sink,
-                   const void* sinks, int64_t k_ld, int64_t v_ld, int gate_kind, int dtype, void* stream) {
+                   const void* sinks, int64_t k_ld, int64_t v_ld, int gate_kind, const lv_attn_extras* extras, int dtype,
+                   void* stream) {
   if (T == 0) return 0;
   if (keep_first < 0 || chunk < 0 || (P > 0 && (keep_first > 0 || chunk > 0)))
     return fail(-1, "lv_masked_attn: kept first tokens and chunks do not combine with pooled blocks");
@@ -322,13 +334,19 @@ int lv_masked_attn(const void* q, const void* k_cache, const void* v_cache, cons
     return fail(-1, "lv_window_pool_attn: gate kind %d", gate_kind);
   const int gate_dv = gate_kind == LV_MIX_GATE_PER_HEAD ? 1 : Dv;
   if (gate != nullptr && ld_gate < static_cast<int64_t>(H) * gate_dv) return fail(-1, "lv_window_pool_attn: gate stride");
+  const bool extended = extras != nullptr && (extras->key_scale != nullptr || extras->dist_bias != nullptr);
+  if (extended && (P > 0 || softcap > 0.0f || (extras->dist_bias != nullptr && extras->bias_len <= 0)))
+    return fail(-1, "lv_masked_attn: key factors and distance biases combine with neither pooled blocks nor a softcap");
+  const int64_t out_ld = extras != nullptr && extras->out_ld > 0 ? extras->out_ld : static_cast<int64_t>(H) * Dv;
+  if (out_ld < static_cast<int64_t>(H) * Dv) return fail(-1, "lv_masked_attn: output stride");
   const bool wide = Dv > 4 * kWave;
   const int kMaxRep = wide ? 4 : 8;
   const int rep = H / G;
   WindowAttnParams p{q, k_cache, v_cache, kp, vp, gate, ld_gate, gate_dv, out, cu_q, ctx_lens, tok_seq, block_tables,
                      bt_stride, H, G, D, Dv, page, window, P, P > 0 ? (page + P - 1) / P : 0, scale,
                      has_sink ? 1.0f : 0.0f, k_ld, v_ld, has_sink ? 0.0f : -1e30f, keep_first, chunk,
-                     static_cast<const float*>(sinks), softcap};
+                     static_cast<const float*>(sinks), softcap, extended ? static_cast<const float*>(extras->key_scale) : nullptr,
+                     extended ? static_cast<const float*>(extras->dist_bias) : nullptr, extended ? extras->bias_len : 0, out_ld};
   const size_t shm = sizeof(float) * (static_cast<size_t>(kMaxRep) * D + 4 * kMaxRep * kWave +
                                       4 * static_cast<size_t>(kMaxRep) * Dv + 4 * kMaxRep * 2);
   if (shm > 64 * 1024) return fail(-2, "lv_window_pool_attn: head sizes %d / %d need %zu bytes of LDS", D, Dv, shm);

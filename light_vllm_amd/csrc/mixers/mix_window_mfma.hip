@@ -13,7 +13,9 @@
 //   O^T += V^T P^T  takes the probabilities of two 16-key blocks as its B operand exactly as they lie (keys x
 //                 queries), with A = V^T read as two 8-byte runs of keys from the 64-entry V tile that the four
 //                 waves stage TRANSPOSED in LDS together.
-// The sink is the initial state of the running softmax: maximum 0, sum 1.
+// The sink is the initial state of the running softmax: maximum 0 (or the head's learned number), sum 1.
+// Extended form: a tile's key factors (norms kept beside unnormed keys) and the heads' distance biases sit in LDS; a score becomes
+// product * scale * factor + bias before the softmax.
 #include "mix_common.h"
 
 namespace lvmix {
@@ -38,14 +40,21 @@ struct WindowMfmaParams {
   int keep_first;      // positions below this are seen from everywhere; they take the place of the pooled tiles (P == 0)
   int chunk;           // > 0: a query sees its own chunk of that many positions (counted from 0) up to itself; no window
   const float* sinks;  // [H] or NULL: a learned score per query head in place of the sink's 0
-  float cap_in, cap;   // CAP form: scores pass cap * tanh(product * cap_in), cap_in = scale / cap
+  float cap_in, cap;   // kCapped: scores pass cap * tanh(product * cap_in), cap_in = scale / cap
+  const float* key_scale;   // kExtended: [pages, page, G] or NULL, a factor on the score of every cached key
+  const float* dist_bias;   // kExtended: [H, bias_len] or NULL, added to the score at distance min(pos - key, bias_len - 1)
+  int bias_len;
+  int64_t out_ld;      // elements between the output rows of two tokens
 };
+
+enum ScoreForm { kPlain = 0, kCapped = 1, kExtended = 2 };
 
 constexpr int kTileQ = 16;
 constexpr int kTileK = 64;
 constexpr int kMaxK32 = 8;     // D <= 256: 32-wide steps over D (template K32: 4 up to D = 128), plus one 16-wide when D % 32 == 16
 constexpr int kLdk = kTileK + 4; // row stride (in keys) of the transposed V tile: rows stay 8-byte aligned
 constexpr int kMaxDvb = 16;    // Dv <= 256
+constexpr int kBiasLds = 1024; // distance biases of a head up to this many are copied to LDS (longer tables are read from memory)
 constexpr int kBtCache = 2048; // page ids of a sequence kept in LDS (longer sequences look them up in memory)
 
 // n / d for 0 <= n < 2^31 with magic = floor(2^32 / d) (0xffffffff for d = 1): the estimate is the quotient or one
@@ -70,7 +79,7 @@ __device__ __forceinline__ float fast_tanh(float x) { return 1.0f - 2.0f * __bui
 // many tiles hide latency by occupancy instead, and every register counts there: with the 32 registers of a V tile held
 // ahead the kernel fell from two waves a SIMD to one and ran 1.7x slower; K32 and DVB size the fragment arrays for the
 // head sizes at hand for the same reason.
-template <bool AHEAD, int K32, int DVB, bool CAP>
+template <bool AHEAD, int K32, int DVB, int FORM>
 __global__ __launch_bounds__(256, (AHEAD || DVB > 8) ? 1 : 4) void window_pool_mfma_kernel(WindowMfmaParams p) {
   extern __shared__ uint16_t vs[];                      // V^T tile [Dv][kLdk]
   const int wave = threadIdx.x / kWave, lane = threadIdx.x % kWave;
@@ -106,6 +115,20 @@ __global__ __launch_bounds__(256, (AHEAD || DVB > 8) ? 1 : 4) void window_pool_m
     __syncthreads();
   }
   auto bt = [&](int idx) { return bt_cached ? bt_lds[idx] : bt_global[idx]; };
+  // kExtended: the tile's key factors and the distance biases of the workgroup's heads, behind the V tile
+  float* ks_lds = reinterpret_cast<float*>(vs + Dv * kLdk);                // [kTileK]
+  float* bias_lds = ks_lds + kTileK;                                       // [4][bias_len]
+  const float* bias_h = nullptr;
+  bool bias_cached = false;
+  if constexpr (FORM == kExtended) {
+    if (p.dist_bias != nullptr) {
+      bias_cached = p.bias_len <= kBiasLds;
+      bias_h = p.dist_bias + static_cast<int64_t>(h) * p.bias_len;
+      if (bias_cached)
+        for (int x = lane; x < p.bias_len; x += kWave) bias_lds[wave * p.bias_len + x] = bias_h[x];   // read by this wave alone
+    }
+    if (p.key_scale == nullptr && threadIdx.x < kTileK) ks_lds[threadIdx.x] = 1.0f;                 // read behind the first barrier
+  }
 
   bf16x8_t qf[K32];
   bf16x4_t qtail = bf16x4_t{0, 0, 0, 0};
@@ -159,6 +182,14 @@ __global__ __launch_bounds__(256, (AHEAD || DVB > 8) ? 1 : 4) void window_pool_m
 
   // V rows of a tile: consecutive threads take consecutive 8-byte segments of a row (whole cache lines per load
   // instruction). AHEAD: all of a thread's loads are issued together, one tile ahead of their use, and wait in registers.
+  // kExtended: the key factor of entry e of the token tiles or of the kept first tokens
+  auto key_factor = [&](int tile, int e) {
+    const int ec = min(e, tile < npt ? nbmax - 1 : i1);
+    const int pj = fdiv(ec, page, p.m_page);
+    return p.key_scale[(static_cast<int64_t>(bt(pj)) * page + (ec - pj * page)) * p.G + g];
+  };
+  const bool keyed = FORM == kExtended && p.key_scale != nullptr && threadIdx.x < kTileK;
+  float ksreg = 1.0f;
   uint2 vreg[AHEAD ? DVB : 1];
   const uint16_t* knext[4];
   auto prefetch = [&](int tile) {
@@ -178,6 +209,7 @@ __global__ __launch_bounds__(256, (AHEAD || DVB > 8) ? 1 : 4) void window_pool_m
       const uint16_t* unused;
       entry_rows(tile, e0 + kb * 16 + ln, knext[kb], unused);
     }
+    if (keyed) ksreg = key_factor(tile, e0 + threadIdx.x);
   };
   auto store_v = [&](uint16_t* dst, uint2 v4) {
     dst[0] = static_cast<uint16_t>(v4.x & 0xffffu);
@@ -226,7 +258,9 @@ __global__ __launch_bounds__(256, (AHEAD || DVB > 8) ? 1 : 4) void window_pool_m
       }
 #pragma unroll
       for (int kb = 0; kb < 4; ++kb) kcur[kb] = knext[kb];
+      if (keyed) ks_lds[threadIdx.x] = ksreg;
     } else {
+      if (keyed) ks_lds[threadIdx.x] = key_factor(tile, e0 + threadIdx.x);
       for (int c = threadIdx.x; c < kTileK * nseg; c += blockDim.x) {
         const int row = fdiv(c, nseg, p.m_nseg), seg = c - row * nseg;
         const uint16_t *kr_, *vr_;
@@ -256,13 +290,27 @@ __global__ __launch_bounds__(256, (AHEAD || DVB > 8) ? 1 : 4) void window_pool_m
         if (tail16)
           acc = __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(
               AHEAD ? ktail[kb] : *reinterpret_cast<const bf16x4_t*>(krow + 32 * nk32 + 4 * lg), qtail, acc, 0, 0, 0);
+        float4 ks = float4{1.0f, 1.0f, 1.0f, 1.0f};
+        if constexpr (FORM == kExtended) ks = *reinterpret_cast<const float4*>(ks_lds + kb * 16 + 4 * lg);
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
           const int ke = e0 + kb * 16 + 4 * lg + i;                         // the key of result row 4*lg + i
           bool vis = ke < e_end;
           if (phase == 0) vis = vis && (P == 0 || ke * P + P - 1 <= pos - W);
           else vis = vis && ke <= pos && ((chunk > 0 ? ke >= cstart : pos - ke < W) || ke < keep);
-          s[kb][i] = vis ? (CAP ? p.cap * fast_tanh(acc[i] * p.cap_in) : acc[i] * p.scale) : -INFINITY;
+          float sc;
+          if constexpr (FORM == kCapped) {
+            sc = p.cap * fast_tanh(acc[i] * p.cap_in);
+          } else if constexpr (FORM == kExtended) {
+            sc = acc[i] * (p.scale * (i == 0 ? ks.x : (i == 1 ? ks.y : (i == 2 ? ks.z : ks.w))));
+            if (bias_h != nullptr) {
+              const int dist = min(max(pos - ke, 0), p.bias_len - 1);
+              sc += bias_cached ? bias_lds[wave * p.bias_len + dist] : bias_h[dist];
+            }
+          } else {
+            sc = acc[i] * p.scale;
+          }
+          s[kb][i] = vis ? sc : -INFINITY;
         }
       }
       if (AHEAD && tile + 1 < t_end) fetch_k();                            // in flight across the softmax, PV and the barriers
@@ -322,7 +370,7 @@ __global__ __launch_bounds__(256, (AHEAD || DVB > 8) ? 1 : 4) void window_pool_m
     return;
   }
   const float inv = l > 0.0f ? 1.0f / l : 0.0f;
-  uint16_t* orow = p.out + (t * p.H + h) * Dv;
+  uint16_t* orow = p.out + t * p.out_ld + static_cast<int64_t>(h) * Dv;
   const uint16_t* grow = p.gate != nullptr ? p.gate + t * p.ld_gate + static_cast<int64_t>(h) * p.gate_dv : nullptr;
   const int gstep = p.gate_dv > 1 ? 1 : 0;
 #pragma unroll
@@ -342,7 +390,7 @@ __global__ __launch_bounds__(256, (AHEAD || DVB > 8) ? 1 : 4) void window_pool_m
 // One wave per (token, query head): combines the splits' partials (each with its own running maximum), applies the gate.
 __global__ __launch_bounds__(256) void window_pool_merge_kernel(const float* __restrict__ ws, const uint16_t* __restrict__ gate,
                                                                 int64_t ld_gate, int gate_dv, uint16_t* __restrict__ out,
-                                                                int64_t items, int H, int Dv, int nsplit, float m0,
+                                                                int64_t items, int H, int Dv, int nsplit, int64_t out_ld, float m0,
                                                                 const float* __restrict__ sinks) {
   const int wave = threadIdx.x / kWave, lane = threadIdx.x % kWave;
   const int64_t item = static_cast<int64_t>(blockIdx.x) * (blockDim.x / kWave) + wave;
@@ -362,7 +410,7 @@ __global__ __launch_bounds__(256) void window_pool_merge_kernel(const float* __r
     if (gate != nullptr)
       val *= sigmoidf_(__builtin_bit_cast(float, static_cast<uint32_t>(gate[t * ld_gate + static_cast<int64_t>(h) * gate_dv +
                                                                             (gate_dv > 1 ? dv : 0)]) << 16));
-    out[item * Dv + dv] = static_cast<uint16_t>(bf16_bits(val));
+    out[t * out_ld + static_cast<int64_t>(h) * Dv + dv] = static_cast<uint16_t>(bf16_bits(val));
   }
 }
 
@@ -380,7 +428,7 @@ extern "C" int lv_window_pool_attn_mfma(const void* q, const void* k_cache, cons
                                         int64_t v_ld, int gate_kind, void* stream) {
   return lv_masked_attn_mfma(q, k_cache, v_cache, kp, vp, gate, ld_gate, out, cu_q, ctx_lens, block_tables, bt_stride, B,
                              max_new_tokens, H, G, D, Dv, page, window, 0, 0, P, scale, 0.0f, has_sink, nullptr, nsplit, workspace, T,
-                             k_ld, v_ld, gate_kind, stream);
+                             k_ld, v_ld, gate_kind, nullptr, stream);
 }
 
 extern "C" int lv_masked_attn_mfma(const void* q, const void* k_cache, const void* v_cache, const void* kp, const void* vp,
@@ -388,7 +436,7 @@ extern "C" int lv_masked_attn_mfma(const void* q, const void* k_cache, const voi
                                    const int32_t* block_tables, int bt_stride, int B, int max_new_tokens, int H, int G, int D,
                                    int Dv, int page, int window, int keep_first, int chunk, int P, float scale, float softcap, int has_sink,
                                    const void* sinks, int nsplit, void* workspace, int64_t T, int64_t k_ld, int64_t v_ld,
-                                   int gate_kind, void* stream) {
+                                   int gate_kind, const lv_attn_extras* extras, void* stream) {
   if (B == 0 || max_new_tokens <= 0) return 0;
   if (keep_first < 0 || chunk < 0 || (P > 0 && (keep_first > 0 || chunk > 0)))
     return fail(-1, "lv_masked_attn_mfma: kept first tokens and chunks do not combine with pooled blocks");
@@ -410,6 +458,11 @@ extern "C" int lv_masked_attn_mfma(const void* q, const void* k_cache, const voi
   if (k_ld < static_cast<int64_t>(G) * D || v_ld < static_cast<int64_t>(G) * Dv || k_ld % 8 != 0 || v_ld % 4 != 0 ||
       (reinterpret_cast<uintptr_t>(k_cache) & 15) != 0 || (reinterpret_cast<uintptr_t>(v_cache) & 7) != 0)
     return fail(-1, "lv_window_pool_attn_mfma: row strides or alignment of the caches");
+  const bool extended = extras != nullptr && (extras->key_scale != nullptr || extras->dist_bias != nullptr);
+  if (extended && (P > 0 || softcap > 0.0f || (extras->dist_bias != nullptr && extras->bias_len <= 0)))
+    return fail(-1, "lv_masked_attn_mfma: key factors and distance biases combine with neither pooled blocks nor a softcap");
+  const int64_t out_ld = extras != nullptr && extras->out_ld > 0 ? extras->out_ld : static_cast<int64_t>(H) * Dv;
+  if (out_ld < static_cast<int64_t>(H) * Dv) return fail(-1, "lv_masked_attn_mfma: output stride");
   const float m0 = has_sink ? 0.0f : -1e30f;
   const int rep = H / G;
   const int ngroups = (rep + 3) / 4;
@@ -420,31 +473,35 @@ extern "C" int lv_masked_attn_mfma(const void* q, const void* k_cache, const voi
                      P > 0 ? (page + P - 1) / P : 0, ngroups, scale, has_sink ? 1.0f : 0.0f,
                      magic(page), magic(P > 0 ? P : 1), magic(Dv / 4), nsplit > 1 ? nsplit : 1, static_cast<float*>(workspace),
                      k_ld, v_ld, m0, keep_first, chunk, static_cast<const float*>(sinks), softcap > 0.0f ? scale / softcap : 0.0f,
-                     softcap};
+                     softcap, extended ? static_cast<const float*>(extras->key_scale) : nullptr,
+                     extended ? static_cast<const float*>(extras->dist_bias) : nullptr, extended ? extras->bias_len : 0, out_ld};
   if (nsplit > 1 && (max_new_tokens > kTileQ || workspace == nullptr || T <= 0))
     return fail(-1, "lv_window_pool_attn_mfma: key splits need one query tile per sequence and a workspace");
-  const size_t shm = static_cast<size_t>(Dv) * kLdk * sizeof(uint16_t);
+  size_t shm = static_cast<size_t>(Dv) * kLdk * sizeof(uint16_t);
+  if (extended) shm += sizeof(float) * (kTileK + (p.dist_bias != nullptr && p.bias_len <= kBiasLds ? 4 * static_cast<size_t>(p.bias_len) : 0));
   dim3 grid(nsplit > 1 ? nsplit : (max_new_tokens + kTileQ - 1) / kTileQ, G * ngroups, B), block(256);
   hipStream_t st = as_stream(stream);
   const bool small = D <= 128 && Dv <= 128;
-#define LVMIX_ATT(AHEAD)                                                                                  \
-  do {                                                                                                    \
-    if (softcap > 0.0f) {                                                                                 \
-      if (small) window_pool_mfma_kernel<AHEAD, 4, 8, true><<<grid, block, shm, st>>>(p);                 \
-      else window_pool_mfma_kernel<AHEAD, kMaxK32, kMaxDvb, true><<<grid, block, shm, st>>>(p);           \
-    } else {                                                                                              \
-      if (small) window_pool_mfma_kernel<AHEAD, 4, 8, false><<<grid, block, shm, st>>>(p);                \
-      else window_pool_mfma_kernel<AHEAD, kMaxK32, kMaxDvb, false><<<grid, block, shm, st>>>(p);          \
-    }                                                                                                     \
+#define LVMIX_ATT_FORM(AHEAD, FORM)                                                               \
+  do {                                                                                            \
+    if (small) window_pool_mfma_kernel<AHEAD, 4, 8, FORM><<<grid, block, shm, st>>>(p);           \
+    else window_pool_mfma_kernel<AHEAD, kMaxK32, kMaxDvb, FORM><<<grid, block, shm, st>>>(p);     \
+  } while (0)
+#define LVMIX_ATT(AHEAD)                                     \
+  do {                                                       \
+    if (softcap > 0.0f) LVMIX_ATT_FORM(AHEAD, kCapped);      \
+    else if (extended) LVMIX_ATT_FORM(AHEAD, kExtended);     \
+    else LVMIX_ATT_FORM(AHEAD, kPlain);                      \
   } while (0)
   if (max_new_tokens <= kTileQ) LVMIX_ATT(true);
   else LVMIX_ATT(false);
 #undef LVMIX_ATT
+#undef LVMIX_ATT_FORM
   if (nsplit > 1) {
     const int64_t items = T * H;
     window_pool_merge_kernel<<<dim3(static_cast<unsigned>((items + 3) / 4)), block, 0, st>>>(
         static_cast<const float*>(workspace), static_cast<const uint16_t*>(gate), ld_gate, gate_dv,
-        static_cast<uint16_t*>(out), items, H, Dv, nsplit, m0, static_cast<const float*>(sinks));
+        static_cast<uint16_t*>(out), items, H, Dv, nsplit, out_ld, m0, static_cast<const float*>(sinks));
   }
   return launched("lv_window_pool_attn_mfma");
 }

@@ -45,19 +45,19 @@ class PolyNorm(nn.Module):
 
 class GatedAct(nn.Module):
     """act(gate) * up over the [gate | up] halves of the last dim; act: "gelu_tanh" (0.5 z (1 + tanh(sqrt(2/pi) (z +
-    0.044715 z^3)))), "gelu" (the exact form) or "relu2"."""
+    0.044715 z^3)))), "gelu" (the exact form), "relu" or "relu2"."""
 
     def __init__(self, act: str = "gelu_tanh"):
         super().__init__()
         assert act in mix_ops.ACTS
         self.act = act
 
-    def forward(self, x: torch.Tensor) -> torch.Tensor:
-        return mix_ops.glu_act(x, self.act)
+    def forward(self, x: torch.Tensor, out: torch.Tensor | None = None) -> torch.Tensor:
+        return mix_ops.glu_act(x, self.act, out)
 
 
 class Act(nn.Module):
-    """The activation without a gate: "relu2", "gelu", "gelu_tanh" or "tanh"."""
+    """The activation without a gate: "relu2", "relu", "gelu", "gelu_tanh" or "tanh"."""
 
     def __init__(self, act: str = "relu2"):
         super().__init__()

@@ -14,9 +14,18 @@ as two batched GEMMs. A decoded token therefore reads kv_rank + rot_dim numbers 
 instead of heads * (dim + vdim), and one attention kernel serves prompts, portions and single tokens:
 the paged windowed kernel with one kv head, a window no sequence reaches, no pooled blocks and no sink.
 
-The output gate is one number per head (`gate="head"`) or one per output channel (`gate="channel"`).
-Rotation: the first rot_dims entries of the rot_dim-wide positional part, entries i and i + rot_dims/2
-form a pair, angle = position * base^(-2i/rot_dims); rot_dim = 0 gives position-free attention.
+The output gate is one number per head (`gate="head"`), one per output channel (`gate="channel"`), or absent (None).
+Rotation: the first rot_dims entries of the rot_dim-wide positional part, entries i and i + rot_dims/2 (or, with `interleaved`, 2i
+and 2i + 1) form a pair, angle = position * base^(-2i/rot_dims), frequencies optionally rescaled and cosines and sines multiplied by
+a factor (mix_ops.rotary_inv_freq, rotary_magnitude); rot_dim = 0 gives position-free attention.
+
+With `window` a position sees itself and the window - 1 tokens before it; with `sink` the softmax denominator of head h also holds
+exp(sink_h), a learned number.
+
+q_rank = None: queries come straight from the layer's input, q = W_q h. One launch then norms and rotates everything that is
+rotated or cached (mix_ops.latent_store), and both batched GEMMs write where the next step reads. Such a module can be built
+`fused`: its input and output projections belong to the caller, who passes the columns of a wider projection and the place of the
+per-head outputs in a wider row (layers.parallel_block).
 """
 from __future__ import annotations
 
@@ -34,29 +43,40 @@ NO_WINDOW = 1 << 30       # a window no sequence reaches: plain causal attention
 class LatentAttention(nn.Module):
     uses_pages = True
 
-    def __init__(self, width: int, heads: int, dim: int, vdim: int, q_rank: int, kv_rank: int, scale: float,
-                 rot_dim: int = 0, rot_dims: int = 0, rot_base: float = 10000.0, gate: str = "head",
-                 norm_eps: float = 1e-6, share: "LatentAttention | None" = None):
+    def __init__(self, width: int, heads: int, dim: int, vdim: int, q_rank: int | None, kv_rank: int, scale: float,
+                 rot_dim: int = 0, rot_dims: int = 0, rot_base: float = 10000.0, gate: str | None = "head",
+                 norm_eps: float = 1e-6, share: "LatentAttention | None" = None, interleaved: bool = False,
+                 rot_scaling: dict | None = None, window: int = NO_WINDOW, sink: bool = False, fused: bool = False):
         super().__init__()
         assert tp_size() == 1, "latent attention is not sharded: run it with tensor_parallel_size 1"
-        assert gate in ("head", "channel") and 0 <= rot_dims <= rot_dim and rot_dims % 2 == 0
+        assert gate in ("head", "channel", None) and 0 <= rot_dims <= rot_dim and rot_dims % 2 == 0 and window >= 1
+        if q_rank is None:
+            assert gate is None, "queries straight from the input come without an output gate"
+        else:
+            assert not (fused or interleaved or rot_scaling) and gate is not None
         self.H, self.Dn, self.Dr, self.Dv, self.Rq, self.R = heads, dim, rot_dim, vdim, q_rank, kv_rank
         self.rot_dims, self.rot_base, self.scale, self.norm_eps = rot_dims, float(rot_base), float(scale), norm_eps
+        self.interleaved, self.rot_scaling, self.window = interleaved, rot_scaling, window
         self.gate_per_channel = gate == "channel"
-        self.sizes = [q_rank, kv_rank + rot_dim, heads * vdim if self.gate_per_channel else heads]   # dq | dkv | gate
+        self.out_size = heads * vdim
+        if q_rank is None:
+            self.sizes = [heads * (dim + rot_dim), kv_rank + rot_dim]                                    # q | dkv
+        else:
+            self.sizes = [q_rank, kv_rank + rot_dim, heads * vdim if self.gate_per_channel else heads]   # dq | dkv | gate
         if share is None:
             f32 = dict(dtype=torch.float32)
-            self.in_proj = MergedColumnParallelLinear(width, self.sizes, bias=False)
-            self.uq = ColumnParallelLinear(q_rank, heads * (dim + rot_dim), bias=False)
+            self.in_proj = None if fused else MergedColumnParallelLinear(width, self.sizes, bias=False)
+            self.uq = ColumnParallelLinear(q_rank, heads * (dim + rot_dim), bias=False) if q_rank is not None else None
             self.uk = nn.Parameter(torch.empty(heads, dim, kv_rank))        # W_uk per head, [dim, kv_rank]
-            self.uv = nn.Parameter(torch.empty(heads, vdim, kv_rank))       # W_uv per head, [vdim, kv_rank]
-            self.o_proj = RowParallelLinear(heads * vdim, width, bias=False)
-            self.q_norm_weight = nn.Parameter(torch.ones(q_rank, **f32))
+            self.uv = nn.Parameter(torch.empty(heads, kv_rank, vdim))       # W_uv per head, transposed: [kv_rank, vdim]
+            self.o_proj = None if fused else RowParallelLinear(heads * vdim, width, bias=False)
+            self.q_norm_weight = nn.Parameter(torch.ones(q_rank, **f32)) if q_rank is not None else None
             self.kv_norm_weight = nn.Parameter(torch.ones(kv_rank, **f32))
+            self.sink = nn.Parameter(torch.zeros(heads, **f32)) if sink else None
         else:       # the same weights as another layer; cache and position in the model are this layer's own
             assert (share.sizes, share.H, share.Dn, share.Dr, share.Dv) == (self.sizes, heads, dim, rot_dim, vdim)
             self.in_proj, self.uq, self.uk, self.uv, self.o_proj = share.in_proj, share.uq, share.uk, share.uv, share.o_proj
-            self.q_norm_weight, self.kv_norm_weight = share.q_norm_weight, share.kv_norm_weight
+            self.q_norm_weight, self.kv_norm_weight, self.sink = share.q_norm_weight, share.kv_norm_weight, share.sink
         self.inv_freq = None          # f32 [rot_dims/2], made with the cache
         self.cache = torch.tensor([])  # [pages, page, kv_rank + rot_dim]; bound by the runner
 
@@ -66,10 +86,21 @@ class LatentAttention(nn.Module):
 
     def bind_cache(self, num_blocks: int, block_size: int, num_slots: int, device, dtype) -> None:
         self.cache = torch.zeros(num_blocks, block_size, self.R + self.Dr, dtype=dtype, device=device)
-        self.inv_freq = mix_ops.rotary_inv_freq(max(self.rot_dims, 2), self.rot_base, device)
+        self.inv_freq = mix_ops.rotary_inv_freq(max(self.rot_dims, 2), self.rot_base, device, self.rot_scaling)
+        self.magnitude = mix_ops.rotary_magnitude(self.rot_scaling)
 
-    def forward(self, h: torch.Tensor) -> torch.Tensor:
+    def _attend(self, q_abs: torch.Tensor, step) -> torch.Tensor:
+        """Per-head weighted sums of the cached latents, [T, H * R]."""
+        rows = self.cache.unsqueeze(2)                                                              # [pages, page, 1, R + Dr]
+        return mix_ops.window_pool_attention(q_abs, rows, rows[..., :self.R], None, None, None, step, self.H, 1, self.R + self.Dr,
+                                             self.R, self.window, 0, self.scale, has_sink=False, sinks=self.sink)
+
+    def forward(self, h: torch.Tensor, proj: torch.Tensor | None = None, col0: int = 0, out: torch.Tensor | None = None) -> torch.Tensor:
+        """proj, col0: a projection of h computed by the caller whose columns from col0 on are this mixer's. A fused module writes
+        the per-head outputs [T, out_size] into `out` and returns that."""
         step = get_context().ragged
+        if self.Rq is None:
+            return self._forward_direct(h, step, proj, col0, out)
         T, H, R, Dn, Dr = h.size(0), self.H, self.R, self.Dn, self.Dr
         proj = self.in_proj(h)
         cq = mix_ops.latent_prep(proj, 0, self.Rq, self.q_norm_weight, self.kv_norm_weight, self.inv_freq, self.cache,
@@ -77,9 +108,21 @@ class LatentAttention(nn.Module):
         q = self.uq(cq)
         q_lat = torch.bmm(q.view(T, H, Dn + Dr)[:, :, :Dn].transpose(0, 1), self.uk)              # [H, T, R]
         q_abs = mix_ops.latent_q_finish(q, q_lat, self.inv_freq, step, H, Dn, Dr, R, self.rot_dims)
-        rows = self.cache.unsqueeze(2)                                                              # [pages, page, 1, R + Dr]
-        o_lat = mix_ops.window_pool_attention(q_abs, rows, rows[..., :R], None, None, None, step, H, 1, R + Dr, R,
-                                              NO_WINDOW, 0, self.scale, has_sink=False)
-        o = torch.bmm(o_lat.view(T, H, R).transpose(0, 1), self.uv.transpose(1, 2))                 # [H, T, Dv]
+        o_lat = self._attend(q_abs, step)
+        o = torch.bmm(o_lat.view(T, H, R).transpose(0, 1), self.uv)                                 # [H, T, Dv]
         gate = proj[:, self.sizes[0] + self.sizes[1]:]
         return self.o_proj(mix_ops.latent_out_gate(o, gate, self.gate_per_channel))
+
+    def _forward_direct(self, h, step, proj, col0, out):
+        T, H, R, Dn, Dr = h.size(0), self.H, self.R, self.Dn, self.Dr
+        if proj is None:
+            proj, col0 = self.in_proj(h), 0
+        q_abs = torch.empty(T, H, R + Dr, dtype=h.dtype, device=h.device)
+        mix_ops.latent_store(proj, col0, col0 + self.sizes[0], self.kv_norm_weight, self.inv_freq, self.magnitude, q_abs, self.cache,
+                             step, H, Dn, Dr, R, self.rot_dims, self.interleaved, self.norm_eps)
+        q = proj[:, col0:col0 + self.sizes[0]].view(T, H, Dn + Dr)
+        torch.bmm(q[:, :, :Dn].transpose(0, 1), self.uk, out=q_abs[:, :, :R].transpose(0, 1))
+        o_lat = self._attend(q_abs.view(T, H * (R + Dr)), step)
+        o = out if out is not None else torch.empty(T, H * self.Dv, dtype=h.dtype, device=h.device)
+        torch.bmm(o_lat.view(T, H, R).transpose(0, 1), self.uv, out=o.view(T, H, self.Dv).transpose(0, 1))
+        return o if self.o_proj is None else self.o_proj(o)

@@ -10,6 +10,9 @@ ctx_lens [B], slots [B], tok_seq [T], block_tables [B, n] and the same lengths a
 """
 from __future__ import annotations
 
+import ctypes
+import math
+
 import torch
 import torch.nn.functional as F
 
@@ -395,7 +398,8 @@ def pool_update(k_cache, v_cache, kp, vp, step, G, D, Dv, P):
 
 
 def window_pool_attention(q, k_cache, v_cache, kp, vp, gate, step, H, G, D, Dv, window, P, scale, has_sink=True,
-                          gate_per_head=False, keep_first=0, chunk=0, sinks=None, softcap=0.0):
+                          gate_per_head=False, keep_first=0, chunk=0, sinks=None, softcap=0.0, key_scale=None, dist_bias=None,
+                          out=None):
     """Query at position i attends to cached positions j with 0 <= i - j < window and to the pooled
     entry of every block b with b*P + P - 1 <= i - window, one softmax over both, `has_sink` adding 1
     to its denominator; the result is multiplied by sigmoid(gate) when a gate is given (gate rows hold
@@ -404,14 +408,24 @@ def window_pool_attention(q, k_cache, v_cache, kp, vp, gate, step, H, G, D, Dv, 
     query sees the positions of its own chunk, floor(i / chunk) == floor(j / chunk), j <= i (chunks count from
     position 0 of the sequence). sinks f32 [H]: the denominator of head h holds exp(sinks[h]) instead of 1.
     Neither combines with pooled blocks. softcap > 0: a score s = q.k * scale becomes softcap * tanh(s / softcap).
-    q [T, H*D] contiguous act; returns act [T, H*Dv]. k_cache and v_cache [pages, page, G, D|Dv] may be
+    key_scale f32 [pages, page, G]: the score of a cached key is multiplied by its number as well. dist_bias f32 [H, L]: head h's
+    score at distance n = i - j gets dist_bias[h, min(n, L - 1)] added (after all factors; the sink gets none). These two combine
+    with windows, kept tokens and chunks, not with pooled blocks or a softcap.
+    q [T, H*D] contiguous act; returns act [T, H*Dv], written into `out` (a view with free row stride) when given. k_cache and v_cache [pages, page, G, D|Dv] may be
     views of wider token rows (one cache row serving as key and, in part, as value). A window that no
     sequence reaches, no pool and no sink give plain causal softmax attention."""
     T = q.size(0)
     page = k_cache.size(1)
-    out = torch.empty(T, H * Dv, dtype=q.dtype, device=q.device)
+    if out is None:
+        out = torch.empty(T, H * Dv, dtype=q.dtype, device=q.device)
+    assert out.shape == (T, H * Dv) and out.stride(1) == 1 and out.dtype == q.dtype
     k_ld, v_ld = k_cache.stride(1), v_cache.stride(1)
     assert P == 0 or (keep_first == 0 and chunk == 0)
+    if key_scale is not None or dist_bias is not None:
+        assert P == 0 and softcap == 0.0
+        _f32(key_scale, dist_bias)
+        assert key_scale is None or key_scale.shape == (*k_cache.shape[:2], G)
+        assert dist_bias is None or dist_bias.size(0) == H
     if sinks is not None:
         _f32(sinks)
         assert sinks.numel() == H
@@ -421,6 +435,7 @@ def window_pool_attention(q, k_cache, v_cache, kp, vp, gate, step, H, G, D, Dv, 
         for c, ld, d in ((k_cache, k_ld, D), (v_cache, v_ld, Dv)):
             assert c.stride(3) == 1 and (G == 1 or c.stride(2) == d) and c.stride(0) == page * ld and ld >= G * d
         lib = _mixlib.load()
+        extras = _mixlib.AttnExtras(_p(key_scale), _p(dist_bias), dist_bias.size(1) if dist_bias is not None else 0, out.stride(0))
         if (WINDOW_ATTN_KERNEL == "auto" and q.dtype == torch.bfloat16 and D % 16 == 0 and Dv % 16 == 0
                 and D <= 256 and Dv <= 256 and k_ld % 8 == 0 and v_ld % 4 == 0 and k_cache.data_ptr() % 16 == 0
                 and v_cache.data_ptr() % 8 == 0):
@@ -441,15 +456,15 @@ def window_pool_attention(q, k_cache, v_cache, kp, vp, gate, step, H, G, D, Dv, 
                                                   step.block_tables.stride(0), len(step.host_lens_q),
                                                   max(step.host_lens_q), H, G, D, Dv, page, window, keep_first, chunk, P, scale,
                                                   softcap, int(has_sink), _p(sinks), nsplit, _p(ws), T, k_ld, v_ld,
-                                                  0 if gate_per_head else 1, _stream(q)),
+                                                  0 if gate_per_head else 1, ctypes.byref(extras), _stream(q)),
                           "lv_masked_attn_mfma")
             return out
         _mixlib.check(lib.lv_masked_attn(_p(q), _p(k_cache), _p(v_cache), _p(kp), _p(vp), _p(gate),
                                          gate.stride(0) if gate is not None else 0, _p(out), _p(step.cu_q),
                                          _p(step.ctx_lens), _p(step.tok_seq), _p(step.block_tables),
                                          step.block_tables.stride(0), T, H, G, D, Dv, page, window, keep_first, chunk, P, scale,
-                                         softcap, int(has_sink), _p(sinks), k_ld, v_ld, 0 if gate_per_head else 1, _DT[q.dtype],
-                                         _stream(q)),
+                                         softcap, int(has_sink), _p(sinks), k_ld, v_ld, 0 if gate_per_head else 1,
+                                         ctypes.byref(extras), _DT[q.dtype], _stream(q)),
                       "lv_masked_attn")
         return out
     PP = pooled_slots(page, P)
@@ -470,6 +485,11 @@ def window_pool_attention(q, k_cache, v_cache, kp, vp, gate, step, H, G, D, Dv, 
                 V = torch.cat([vp.view(-1, G, Dv)[prow].float(), V])
             qi = q[q0 + r].float().view(G, rep, D)
             s = torch.einsum("grd,ngd->grn", qi, K) * scale
+            if key_scale is not None:
+                s = s * key_scale.view(-1, G)[rows].t().unsqueeze(1)
+            if dist_bias is not None:
+                seen = torch.tensor(list(range(min(keep_first, j0))) + list(range(j0, i + 1)))
+                s = s + dist_bias[:, (i - seen).clamp(max=dist_bias.size(1) - 1)].view(G, rep, -1)
             if softcap > 0:
                 s = softcap * torch.tanh(s / softcap)
             m = s.max(-1, keepdim=True).values
@@ -492,16 +512,51 @@ def rotary_inv_freq(dims: int, base: float, device, scaling: dict | None = None)
     """f32 [dims/2]: base^(-2i/dims), computed in 64-bit and rounded once. `scaling` (factor, low, high,
     original) rescales by wavelength 2 pi / f: waves shorter than original / high keep their frequency,
     waves longer than original / low get f / factor, and those between are blended linearly in
-    original / wavelength."""
+    original / wavelength. `scaling` with (factor, original, fast, slow) is YaRN's: the pair whose wave turns `t` times over
+    the original length has the fractional index d(t) = dims ln(original / (2 pi t)) / (2 ln base); pairs up to
+    floor(d(fast)) keep their frequency, pairs from ceil(d(slow)) on get f / factor, linear in the index between
+    (rotary_magnitude is its factor on cosines and sines)."""
     i = torch.arange(dims // 2, dtype=torch.float64)
     f = torch.pow(torch.tensor(float(base), dtype=torch.float64), -2.0 * i / dims)
-    if scaling:
+    if scaling and "fast" in scaling:
+        factor, original = float(scaling["factor"]), float(scaling["original"])
+        lo, hi = (dims * math.log(original / (2.0 * math.pi * float(scaling[k]))) / (2.0 * math.log(float(base)))
+                  for k in ("fast", "slow"))
+        lo, hi = max(math.floor(lo), 0), min(math.ceil(hi), dims - 1)
+        ramp = ((i - lo) / max(hi - lo, 0.001)).clamp(0.0, 1.0)
+        f = f / factor * ramp + f * (1.0 - ramp)
+    elif scaling:
         factor, low, high = float(scaling["factor"]), float(scaling["low"]), float(scaling["high"])
         turns = float(scaling["original"]) * f / (2.0 * torch.pi)          # original / wavelength
         blend = ((turns - low) / (high - low)).clamp(0.0, 1.0) if high != low else (turns >= high).double()
         blend = torch.where(turns > high, torch.ones_like(blend), torch.where(turns < low, torch.zeros_like(blend), blend))
         f = (1.0 - blend) * f / factor + blend * f
     return f.float().to(device)
+
+
+def rotary_magnitude(scaling: dict | None) -> float:
+    """What a scaled rotation multiplies its cosines and sines by: 0.1 ln(factor) + 1 for YaRN's kind, else 1."""
+    return 0.1 * math.log(float(scaling["factor"])) + 1.0 if scaling and "fast" in scaling else 1.0
+
+
+def distance_bias(rel: torch.Tensor, far: int, window: int) -> torch.Tensor:
+    """rel [B, H], one bias per bucket and head -> f32 [H, L], the bias at distances 0 .. L - 1; the last entry serves every
+    distance beyond. The first B/2 buckets hold one distance each, the others are spaced by the logarithm up to distance `far`:
+    bucket(n) = min(B - 1, B/2 + floor(ln(n / (B/2)) / ln(far / (B/2)) (B - B/2))). L ends where the last bucket begins or
+    the window does."""
+    B = rel.size(0)
+    half = B // 2
+    assert half >= 1 and far > half, "the buckets' far distance lies within their linear half"
+
+    def bucket(n):
+        return n if n < half else min(B - 1, half + math.floor(math.log(n / half) / math.log(far / half) * (B - half)))
+
+    idx = []
+    for n in range(max(1, min(window, far + 1))):
+        idx.append(bucket(n))
+        if idx[-1] == B - 1:
+            break
+    return rel.float()[torch.tensor(idx, device=rel.device)].t().contiguous()
 
 
 def _rotate(x, pos, inv_freq, dims, interleaved=False):
@@ -608,6 +663,78 @@ def latent_prep(proj, off_q, off_kv, q_w, kv_w, inv_freq, cache, step, Rq, R, Dr
             flat[_token_slot(bt, ctx + r, page)] = rows[q0 + r]
         q0 += n
     return cq
+
+
+def latent_store(proj, off_q, off_kv, kv_w, inv_freq, magnitude, q_out, cache, step, H, Dn, Dr, R, rot_dims, interleaved, eps):
+    """Latent attention whose queries come straight from the layer's input. proj act [T, ld]: H queries of Dn + Dr at column
+    off_q (rotated part last), the key/value latent at off_kv (R wide) followed by the positional key part (Dr wide). Writes
+    [rms_norm(latent) * kv_w | rotated positional part] into each token's row of cache [pages, page, R + Dr], and the rotated
+    query parts into q_out act [T, H, R + Dr] behind the R entries of every head, which the caller fills. Pairs of rotated
+    entries are (i, i + rot_dims/2), or (2i, 2i + 1) with `interleaved`; cosines and sines are multiplied by `magnitude`."""
+    T = proj.size(0)
+    page = cache.size(1)
+    _f32(kv_w, inv_freq)
+    assert cache.is_contiguous() and cache.shape[2] == R + Dr and cache.dtype == proj.dtype
+    assert q_out.is_contiguous() and q_out.shape == (T, H, R + Dr) and q_out.dtype == proj.dtype
+    if proj.is_cuda:
+        assert proj.stride(1) == 1
+        lib = _mixlib.load()
+        _mixlib.check(lib.lv_latent_store(_p(proj), proj.stride(0), off_q, off_kv, _p(kv_w), _p(inv_freq), float(magnitude),
+                                          _p(q_out), _p(cache), _p(step.cu_q), _p(step.ctx_lens), _p(step.tok_seq),
+                                          _p(step.block_tables), step.block_tables.stride(0), T, H, Dn, Dr, R, rot_dims,
+                                          int(interleaved), page, eps, _DT[proj.dtype], _stream(proj)), "lv_latent_store")
+        return
+    pos = _positions(step, proj.device)
+
+    def turned(x):
+        y = _rotate(x, pos, inv_freq, rot_dims, interleaved)
+        return torch.cat([y[..., :rot_dims] * magnitude, y[..., rot_dims:]], -1)
+
+    c = proj[:, off_kv:off_kv + R].float()
+    c = c / torch.sqrt(c.pow(2).mean(-1, keepdim=True) + eps) * kv_w
+    if Dr:
+        q_out[..., R:] = turned(proj[:, off_q:off_q + H * (Dn + Dr)].float().view(T, H, Dn + Dr)[..., Dn:]).to(proj.dtype)
+    rows = torch.cat([c, turned(proj[:, off_kv + R:off_kv + R + Dr].float())], -1).to(cache.dtype)
+    flat = cache.view(-1, R + Dr)
+    q0 = 0
+    for b, (n, ctx) in enumerate(zip(step.host_lens_q, step.host_ctx_lens)):
+        for r in range(n):
+            flat[_token_slot(step.host_block_tables[b], ctx + r, page)] = rows[q0 + r]
+        q0 += n
+
+
+def head_norm_store(proj, off_q, off_k, q_w, cache, key_scale, step, H, G, D, eps):
+    """proj act [T, ld]: H query heads of D at column off_q, G key heads of D at off_k. Every query head is divided by
+    sqrt(mean(head^2) + eps) and multiplied by q_w f32 [D]; keys go to the token's row of cache [pages, page, G, D] as they are,
+    their 1 / sqrt(mean(head^2) + eps) to key_scale f32 [pages, page, G]. A normed key with weight k_w has the product
+    q . (k_w * k * key_scale) = (q * k_w) . k * key_scale with a query, so that one cached row serves as normed key (with k_w folded
+    into q_w) and as unnormed value. Returns the queries, act [T, H*D]."""
+    T = proj.size(0)
+    page = cache.size(1)
+    _f32(q_w, key_scale)
+    assert cache.is_contiguous() and cache.shape[2:] == (G, D) and cache.dtype == proj.dtype
+    assert key_scale.shape == (*cache.shape[:2], G) and q_w.numel() == D
+    q_out = torch.empty(T, H * D, dtype=proj.dtype, device=proj.device)
+    if proj.is_cuda:
+        assert proj.stride(1) == 1
+        lib = _mixlib.load()
+        _mixlib.check(lib.lv_head_norm_store(_p(proj), proj.stride(0), off_q, off_k, _p(q_w), _p(q_out), _p(cache), _p(key_scale),
+                                             _p(step.cu_q), _p(step.ctx_lens), _p(step.tok_seq), _p(step.block_tables),
+                                             step.block_tables.stride(0), T, H, G, D, page, eps, _DT[proj.dtype], _stream(proj)),
+                      "lv_head_norm_store")
+        return q_out
+    q = proj[:, off_q:off_q + H * D].float().view(T, H, D)
+    q_out.copy_((q / torch.sqrt(q.pow(2).mean(-1, keepdim=True) + eps) * q_w).reshape(T, H * D))
+    k = proj[:, off_k:off_k + G * D]
+    inv = 1.0 / torch.sqrt(k.float().view(T, G, D).pow(2).mean(-1) + eps)
+    kc, ks = cache.view(-1, G * D), key_scale.view(-1, G)
+    q0 = 0
+    for b, (n, ctx) in enumerate(zip(step.host_lens_q, step.host_ctx_lens)):
+        for r in range(n):
+            sl = _token_slot(step.host_block_tables[b], ctx + r, page)
+            kc[sl], ks[sl] = k[q0 + r], inv[q0 + r]
+        q0 += n
+    return q_out
 
 
 def latent_q_finish(q, q_lat, inv_freq, step, H, Dn, Dr, R, rot_dims):
@@ -724,27 +851,30 @@ def moe_grouped_ok(h, Fe) -> bool:
     return h.dtype == torch.bfloat16 and h.size(1) % 32 == 0 and Fe % 32 == 0
 
 
-ACTS = {"relu2": 0, "gelu": 1, "gelu_tanh": 2, "tanh": 3}
+ACTS = {"relu2": 0, "gelu": 1, "gelu_tanh": 2, "tanh": 3, "relu": 4}
 
 
 def _act(x, act):
-    """x f32 -> relu(x)^2, exact gelu, the tanh form of gelu, or tanh."""
-    if act == "relu2":
-        return torch.relu(x).pow(2)
+    """x f32 -> relu(x)^2, relu(x), exact gelu, the tanh form of gelu, or tanh."""
+    if act in ("relu", "relu2"):
+        return torch.relu(x) if act == "relu" else torch.relu(x).pow(2)
     if act == "tanh":
         return torch.tanh(x)
     return F.gelu(x, approximate="tanh" if act == "gelu_tanh" else "none")
 
 
-def glu_act(x, act="gelu_tanh"):
-    """x act [T, 2F] = [gate | up] (row stride free) -> act [T, F] = act(gate) * up."""
+def glu_act(x, act="gelu_tanh", out=None):
+    """x act [T, 2F] = [gate | up] (row stride free) -> act [T, F] = act(gate) * up, written into `out` (a view with free row
+    stride) when given."""
     T, F2 = x.shape
     Fh = F2 // 2
-    out = torch.empty(T, Fh, dtype=x.dtype, device=x.device)
+    if out is None:
+        out = torch.empty(T, Fh, dtype=x.dtype, device=x.device)
+    assert out.shape == (T, Fh) and out.stride(1) == 1 and out.dtype == x.dtype
     if x.is_cuda:
         assert x.stride(1) == 1
         lib = _mixlib.load()
-        _mixlib.check(lib.lv_glu_act(_p(x), x.stride(0), _p(out), T, Fh, ACTS[act], _DT[x.dtype], _stream(x)), "lv_glu_act")
+        _mixlib.check(lib.lv_glu_act(_p(x), x.stride(0), _p(out), out.stride(0), T, Fh, ACTS[act], _DT[x.dtype], _stream(x)), "lv_glu_act")
         return out
     out.copy_(_act(x[:, :Fh].float(), act) * x[:, Fh:].float())
     return out
@@ -1312,7 +1442,7 @@ def embed_norm(ids, table, scale, pair_table, buckets, mul_prev, mul_cur, prev_s
 
 
 def unary_act(x, act="relu2"):
-    """act(x) element by element (relu2, gelu, gelu_tanh or tanh), computed in f32, in x's dtype."""
+    """act(x) element by element (relu2, relu, gelu, gelu_tanh or tanh), computed in f32, in x's dtype."""
     out = torch.empty_like(x)
     if x.is_cuda:
         assert x.is_contiguous()
@@ -1321,3 +1451,114 @@ def unary_act(x, act="relu2"):
         return out
     out.copy_(_act(x.float(), act))
     return out
+
+
+# --------------------------------------------------------------------- gated linear recurrence, re-entered residual
+LRU_TILE = 64              # tokens a workgroup of the recurrence takes at a time
+LRU_COLUMNS = 64           # channels of one workgroup
+
+
+def lru_mfma_ok(u, blocks) -> bool:
+    """Whether the matrix-core kernels serve these shapes (bf16, gate matrices in multiples of 32, aligned rows)."""
+    return u.dtype == torch.bfloat16 and (u.size(1) // blocks) % 32 == 0 and u.data_ptr() % 16 == 0 and u.stride(0) % 8 == 0
+
+
+def gated_linear_recurrence(u, y, gate_w, gate_b, rate, state, step, blocks, out=None):
+    """Real-gated linear recurrent unit, channel by channel. u act [T, N] (the convolved branch), y act [T, N] (the other
+    branch before its gelu), row strides free; the N channels are split into `blocks` equal parts of n. gate_w act
+    [blocks, 2, n, n], gate_b f32 [blocks, 2, n], rate f32 [N] (at most 0):
+        r, i = sigmoid(gate_w[b, 0] u_b + gate_b[b, 0]), sigmoid(gate_w[b, 1] u_b + gate_b[b, 1])
+        log a = rate * r;  S <- a S + sqrt(1 - a^2) i u;  out = S gelu_tanh(y)
+    state f32 [slots, N] (taken as zero for a sequence with no context), updated in place; everything from the gates on in f32.
+    Returns act [T, N], written into `out` (a view with free row stride) when given."""
+    T, N = u.shape
+    n = N // blocks
+    _f32(gate_b, rate, state)
+    assert N % blocks == 0 and gate_w.shape == (blocks, 2, n, n) and gate_w.is_contiguous() and gate_b.shape == (blocks, 2, n)
+    assert state.size(1) == N and rate.numel() == N and y.shape == (T, N) and gate_w.dtype == u.dtype == y.dtype
+    if out is None:
+        out = torch.empty(T, N, dtype=u.dtype, device=u.device)
+    assert out.shape == (T, N) and out.stride(1) == 1 and out.dtype == u.dtype
+    if u.is_cuda:
+        assert u.stride(1) == 1 and y.stride(1) == 1
+        lib = _mixlib.load()
+        B, most = len(step.host_lens_q), max(step.host_lens_q)
+        mfma = lru_mfma_ok(u, blocks)
+        nsplit, ws = 1, None
+        if mfma and most > LRU_TILE:
+            # too few workgroups to fill the chip: cut the sequences, whose parts first hand their decays and sums to the later ones
+            columns = blocks * -(-n // LRU_COLUMNS)
+            nsplit = max(1, min(-(-most // LRU_TILE), 512 // (columns * B), 64))
+            if nsplit > 1:
+                ws = torch.empty(B, nsplit, 2, N, dtype=torch.float32, device=u.device)
+        _mixlib.check(lib.lv_gated_linear_recurrence(_p(u), u.stride(0), _p(y), y.stride(0), _p(gate_w), _p(gate_b), _p(rate), _p(state),
+                                                     _p(step.cu_q), _p(step.ctx_lens), _p(step.slots), _p(out), out.stride(0), B, T,
+                                                     most, N, blocks, nsplit, _p(ws), int(mfma), _DT[u.dtype], _stream(u)),
+                      "lv_gated_linear_recurrence")
+        return out
+    uf = u.float()
+    pre = torch.einsum("tbk,bgok->tbgo", uf.view(T, blocks, n), gate_w.float()) + gate_b
+    r, i = torch.sigmoid(pre[:, :, 0]).reshape(T, N), torch.sigmoid(pre[:, :, 1]).reshape(T, N)
+    log_a = rate * r
+    a, x = torch.exp(log_a), torch.sqrt(-torch.expm1(2.0 * log_a)) * i * uf
+    g = F.gelu(y.float(), approximate="tanh")
+    q0 = 0
+    for b, (m, ctx) in enumerate(zip(step.host_lens_q, step.host_ctx_lens)):
+        slot = step.host_slots[b]
+        S = state[slot].clone() if ctx > 0 else torch.zeros(N)
+        for t in range(q0, q0 + m):
+            S = a[t] * S + x[t]
+            out[t] = S * g[t]
+        state[slot] = S
+        q0 += m
+    return out
+
+
+def scaled_embedding(ids, table, scale, want_rows=False, want_split=False):
+    """ids int64 [T] -> (x f32 [T, W] = table[id] * scale, the rows themselves act [T, W] or None, residual_split of x or None)."""
+    T, W = ids.numel(), table.size(1)
+    x = torch.empty(T, W, dtype=torch.float32, device=table.device)
+    rows = torch.empty(T, W, dtype=table.dtype, device=table.device) if want_rows else None
+    split = torch.empty(T, 2 * W, dtype=torch.bfloat16, device=table.device) if want_split else None
+    if table.is_cuda:
+        assert ids.dtype == torch.int64 and ids.is_contiguous() and table.is_contiguous()
+        lib = _mixlib.load()
+        _mixlib.check(lib.lv_scaled_embedding(_p(ids), _p(table), table.size(0), float(scale), _p(x), _p(rows), _p(split), T, W,
+                                              _DT[table.dtype], _stream(table)), "lv_scaled_embedding")
+        return x, rows, split
+    picked = table[ids]
+    x.copy_(picked.float() * scale)
+    if want_rows:
+        rows.copy_(picked)
+    if want_split:
+        split[:, :W] = x
+        split[:, W:] = x - split[:, :W].float()
+    return x, rows, split
+
+
+def residual_split(x, y=None):
+    """x [T, W] f32 += y (act [T, W], may be None) in place; returns bf16 [T, 2W] = [high | low] with high = x rounded and low = x -
+    high rounded: two bf16 numbers that hold the residual to 16 bits of mantissa, as operands of a matrix product."""
+    T, W = x.shape
+    _f32(x)
+    out = torch.empty(T, 2 * W, dtype=torch.bfloat16, device=x.device)
+    if x.is_cuda:
+        assert y is None or (y.is_contiguous() and y.dtype == torch.bfloat16 and y.shape == (T, W))
+        lib = _mixlib.load()
+        _mixlib.check(lib.lv_residual_split(_p(x), _p(y), _p(out), T, W, _stream(x)), "lv_residual_split")
+        return out
+    if y is not None:
+        x.add_(y.float())
+    out[:, :W] = x
+    out[:, W:] = x - out[:, :W].float()
+    return out
+
+
+def mm_f32(a, b_t, add=None):
+    """a act [T, K], b_t act [K, N] -> f32 [T, N] = a b_t (+ add f32 [T, N]), summed and left in f32."""
+    if a.dtype == torch.float32:
+        return torch.mm(a, b_t) if add is None else torch.addmm(add, a, b_t)
+    if a.is_cuda:
+        return torch.mm(a, b_t, out_dtype=torch.float32) if add is None else torch.addmm(add, a, b_t, out_dtype=torch.float32)
+    y = torch.mm(a.float(), b_t.float())
+    return y if add is None else y + add

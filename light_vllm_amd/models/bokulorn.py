@@ -202,7 +202,8 @@ class BokulornForCausalLM(nn.Module):
     # ------------------------------------------------------------------ checkpoint
     def weight_targets(self) -> dict:
         """checkpoint tensor name -> (parameter, where, shape): where is None (the whole parameter), the
-        index of a part of a merged projection, ("rows", offset, size) or ("cols", offset, size)."""
+        index of a part of a merged projection, ("rows", offset, size), ("cols", offset, size), or ("head_transposed",)
+        for a stack of matrices, one per head, that are held transposed."""
         t = {}
 
         def whole(name, param, shape=None):
@@ -238,7 +239,7 @@ class BokulornForCausalLM(nn.Module):
                 whole(p + "mix.dkv.norm", mix.kv_norm_weight)
                 whole(p + "mix.uq", mix.uq.weight)
                 whole(p + "mix.uk", mix.uk, (mix.H * mix.Dn, mix.R))       # head by head: a view of [H, dim, R]
-                whole(p + "mix.uv", mix.uv, (mix.H * mix.Dv, mix.R))
+                t[p + "mix.uv"] = (mix.uv, ("head_transposed",), (mix.H * mix.Dv, mix.R))  # held as [H, R, vdim]
             whole(p + "mix.o", mix.o_proj.weight)
             if layer.mlp is not None:
                 moe = layer.mlp
@@ -267,6 +268,9 @@ class BokulornForCausalLM(nn.Module):
                     param.data.copy_(tensor.reshape(param.shape))
             elif isinstance(where, tuple) and where[0] == "rows":
                 param.data[where[1]:where[1] + where[2]].copy_(tensor)
+            elif isinstance(where, tuple) and where[0] == "head_transposed":
+                H, R, Dv = param.shape
+                param.data.copy_(tensor.view(H, Dv, R).transpose(1, 2))
             elif isinstance(where, tuple):
                 param.data[:, where[1]:where[1] + where[2]].copy_(tensor)
             else:

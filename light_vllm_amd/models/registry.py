@@ -41,6 +41,11 @@ def _feditar():
     return FeditarForCausalLM
 
 
+def _gokolix():
+    from .gokolix import GokolixForCausalLM
+    return GokolixForCausalLM
+
+
 MODELS = {
     "Qwen3ForCausalLM": _qwen3,
     "Kagalorn": _kagalorn,
@@ -48,6 +53,7 @@ MODELS = {
     "Givozen": _givozen,
     "Bisuzen": _bisuzen,
     "Feditar": _feditar,
+    "Gokolix": _gokolix,
 }
 DEFAULT = "Qwen3ForCausalLM"
 

@@ -83,4 +83,4 @@ def test_argument_validation_happens_before_any_launch():
     assert lib.lv_embed_norm(p, p, 8, 1.0, p, 0, 1, 1, p, None, 0, p, p, 1.0, 1e-6, p, p, p, p, p, p, 1, 8, 0, None) == -1   # no buckets
     assert lib.lv_embed_norm(p, p, 8, 1.0, None, 0, 0, 0, None, p, 0, p, p, 1.0, 1e-6, p, p, p, p, p, p, 1, 8, 0, None) == -1   # empty position table
     assert lib.lv_unary_act(p, p, 8, 17, 0, None) == -1
-    assert lib.lv_masked_attn(p, p, p, None, None, None, 0, p, p, p, p, p, 1, 1, 4, 2, 8, 8, 16, 64, 0, 0, 0, 0.5, -1.0, 0, None, 0, 0, 1, 0, None) == -1   # cap
+    assert lib.lv_masked_attn(p, p, p, None, None, None, 0, p, p, p, p, p, 1, 1, 4, 2, 8, 8, 16, 64, 0, 0, 0, 0.5, -1.0, 0, None, 0, 0, 1, None, 0, None) == -1   # cap
