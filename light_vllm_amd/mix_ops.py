@@ -552,7 +552,7 @@ def distance_bias(rel: torch.Tensor, far: int, window: int) -> torch.Tensor:
         return n if n < half else min(B - 1, half + math.floor(math.log(n / half) / math.log(far / half) * (B - half)))
 
     idx = []
-    for n in range(max(1, min(window, far + 1))):
+    for n in range(max(1, min(window, math.ceil(far) + 1))):
         idx.append(bucket(n))
         if idx[-1] == B - 1:
             break

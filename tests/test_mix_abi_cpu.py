@@ -84,3 +84,20 @@ def test_argument_validation_happens_before_any_launch():
     assert lib.lv_embed_norm(p, p, 8, 1.0, None, 0, 0, 0, None, p, 0, p, p, 1.0, 1e-6, p, p, p, p, p, p, 1, 8, 0, None) == -1   # empty position table
     assert lib.lv_unary_act(p, p, 8, 17, 0, None) == -1
     assert lib.lv_masked_attn(p, p, p, None, None, None, 0, p, p, p, p, p, 1, 1, 4, 2, 8, 8, 16, 64, 0, 0, 0, 0.5, -1.0, 0, None, 0, 0, 1, None, 0, None) == -1   # cap
+    # the gated linear recurrence, stored norms, split residuals, extended attention
+    assert lib.lv_gated_linear_recurrence(None, 0, None, 0, None, None, None, None, None, None, None, None, 0, 0, 0, 0, 8, 2, 1, None, 0, 0, None) == 0
+    lru = lambda **kw: [p, kw.get("ldu", 64), p, kw.get("ldy", 64), p, p, p, p, p, p, p, p, 64, 1, 1, 1, 64, kw.get("blocks", 2), kw.get("nsplit", 1),  # noqa: E731
+                        kw.get("ws"), kw.get("mfma", 1), kw.get("dt", 0), None]
+    assert lib.lv_gated_linear_recurrence(*lru(blocks=3)) == -1 and lib.lv_gated_linear_recurrence(*lru(ldu=63)) == -1
+    assert lib.lv_gated_linear_recurrence(*lru(nsplit=2)) == -1 and lib.lv_gated_linear_recurrence(*lru(nsplit=2, ws=p, mfma=0)) == -1    # no workspace; no parts
+    assert lib.lv_gated_linear_recurrence(*lru(blocks=4)) == -1 and lib.lv_gated_linear_recurrence(*lru(dt=1)) == -1     # blocks of 16, f32: not the matrix cores
+    assert lib.lv_gated_linear_recurrence(*lru(ldu=68)) == -1 and lib.lv_gated_linear_recurrence(*lru(ldy=60)) == -1
+    hn = lambda **kw: [p, kw.get("ld", 64), 0, 32, p, p, p, kw.get("ks", p), p, p, p, p, 1, 1, kw.get("H", 4), kw.get("G", 2), 8, 16, 1e-6, 0, None]  # noqa: E731
+    assert lib.lv_head_norm_store(*hn(ld=40)) == -1 and lib.lv_head_norm_store(*hn(H=3)) == -1 and lib.lv_head_norm_store(*hn(ks=None)) == -1
+    ls = lambda **kw: [p, kw.get("ld", 64), 0, 48, p, p, 1.0, p, p, p, p, p, p, 1, 1, 4, 8, 4, kw.get("R", 12), kw.get("rot", 4), 1, 16, 1e-6, 0, None]  # noqa: E731
+    assert lib.lv_latent_store(*ls(R=13)) == -1 and lib.lv_latent_store(*ls(rot=3)) == -1 and lib.lv_latent_store(*ls(rot=6)) == -1
+    assert lib.lv_scaled_embedding(p, p, 0, 1.0, p, None, None, 1, 8, 0, None) == -1 and lib.lv_residual_split(p, None, None, 1, 8, None) == -1
+    assert lib.lv_glu_act(p, 16, p, 7, 1, 8, 4, 0, None) == -1 and lib.lv_glu_act(p, 16, p, 8, 1, 8, 5, 0, None) == -1              # short output rows; unknown act
+    ext = lambda **kw: ctypes.byref(_mixlib.AttnExtras(p, p, kw.get("n", 4), kw.get("ld", 0)))  # noqa: E731
+    for ex, P, cap in ((ext(), 4, 0.0), (ext(), 0, 2.0), (ext(n=0), 0, 0.0), (ext(ld=31), 0, 0.0)):     # pools, a softcap, an empty table, short rows
+        assert lib.lv_masked_attn(p, p, p, p, p, None, 0, p, p, p, p, p, 1, 1, 4, 2, 8, 8, 16, 64, 0, 0, P, 0.5, cap, 0, None, 0, 0, 1, ex, 0, None) == -1
