@@ -1461,6 +1461,209 @@ def feditar_leg(sizes, batch, prompt_len, new_tokens, engine_only=False):
     print(json.dumps(out), flush=True)
 
 
+# --mixers-design gokolix: the Gokolix design (windowed latent attention, windowed attention with distance biases on shared key/value
+# rows, gated linear recurrence; mixer and feed-forward side by side in two GEMMs; a layer in two passes) beside Bisuzen, the
+# closest existing model (windowed attention with sinks, a recurrence in f32, gated feed-forwards, looped layers), at equal width,
+# layer runs, head counts and active feed-forward parameters (three matrices of two thirds of the size instead of two).
+GOKOLIX_SIZES = {
+    "2k": dict(kv_rank=192, rot_dim=64, window=512, rel_rows=32, rel_far=128, conv=4, blocks=16),
+    "4k": dict(kv_rank=192, rot_dim=64, window=512, rel_rows=32, rel_far=128, conv=4, blocks=32),
+}
+
+
+def _gokolix_config(z, kz):
+    from light_vllm_amd.models.gokolix import GokolixConfig
+    H, G, D, Dr = z["heads"], z["kv_heads"], z["dim"], kz["rot_dim"]
+    latent = {"heads": H, "dim": D, "vdim": D, "kv_rank": kz["kv_rank"], "rot_dim": Dr, "scale": (D + Dr) ** -0.5,
+              "mask": {"size": kz["window"]},
+              "rot": {"base": 10000.0, "dims": Dr, "scaling": {"factor": 8.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}
+    att = {"heads": H, "kv_heads": G, "dim": D, "vdim": D, "scale": D ** -0.5, "mask": {"size": kz["window"]},
+           "bias_max": kz["rel_far"], "rel_rows": kz["rel_rows"]}
+    lru = {"width": z["width"], "blocks": kz["blocks"], "conv": kz["conv"]}
+    kinds = [("latent_attention", latent), ("attention", att), ("rglru", lru), ("attention", att)]
+    layers = [{"type": kinds[i % 4][0], "mixer": kinds[i % 4][1], "mlp": {"kind": "dense", "ff": z["ff"] * 2 // 3}}
+              for i in range(z["layers"] - 1)]           # the first one runs twice
+    return GokolixConfig.from_dict({"vocab": z["vocab"], "width": z["width"], "norm": {"eps": 1e-6},
+                                    "embedding": {"scale": z["width"] ** 0.5}, "layers": layers,
+                                    "loop": {"start": 0, "stop": 1, "times": 2}})
+
+
+def _gokolix_kernel_table(z, kz, fz, dev, batch, prompt_len):
+    """Each kernel of the design alone at one layer's shapes (prompt step and decode step), beside the kernel of Bisuzen (or, for
+    the latent attention and the convolution, of Bokulorn and Feditar) that does the like job."""
+    from light_vllm_amd import mix_ops
+    from light_vllm_amd.utils.context import RaggedStep
+    bf = torch.bfloat16
+    W, H, G, D, ff = z["width"], z["heads"], z["kv_heads"], z["dim"], z["ff"] * 2 // 3
+    R, Dr, window, taps, blocks = kz["kv_rank"], kz["rot_dim"], kz["window"], kz["conv"], kz["blocks"]
+    page = 256
+    rows = []
+
+    def step_of(lens_q, ctx):
+        B = len(lens_q)
+        cu, tok = [0], []
+        for b, n_ in enumerate(lens_q):
+            cu.append(cu[-1] + n_)
+            tok += [b] * n_
+        per = -(-(max(ctx) + max(lens_q)) // page)
+        tables = [[b * per + j for j in range(per)] for b in range(B)]
+        i32 = dict(dtype=torch.int32, device=dev)
+        return RaggedStep(torch.tensor(cu, **i32), torch.tensor(ctx, **i32), torch.arange(B, **i32),
+                          torch.tensor(tok, **i32), torch.tensor(tables, **i32), lens_q, ctx, list(range(B)), tables), B * per
+
+    def add(name, phase, fn, nbytes=0, flops=0, like=None, matrix=False):
+        us = _graph_time(fn) * 1e6
+        rec = {"kernel": name, "phase": phase, "us": round(us, 1)}
+        if nbytes:
+            rec["of_hbm_roofline"] = round(nbytes / us / 1e3 / (HBM_BPS / 1e9), 3)
+        if flops:
+            rec["TFLOPs"] = round(flops / us / 1e6, 2)
+            if matrix:
+                rec["of_mfma_roofline"] = round(flops / us / 1e6 / (MFMA_FLOPS / 1e12), 4)
+        if like:
+            rec["like"] = like
+        rows.append(rec)
+
+    def rand(*shape, dtype=bf):
+        return torch.randn(*shape, device=dev, dtype=dtype)
+
+    for phase, lens_q, ctx in (("prompt", [prompt_len] * batch, [0] * batch), ("decode", [1] * batch, [prompt_len] * batch)):
+        step, pages = step_of(lens_q, ctx)
+        T, B = sum(lens_q), len(lens_q)
+        decode = phase == "decode"
+        x, y1, y2 = rand(T, W, dtype=torch.float32), rand(T, W), rand(T, W)
+        nw, alpha = torch.ones(W, device=dev), torch.full((1,), 0.5, device=dev)
+        # embedding, entry of a pass, residual
+        table = rand(z["vocab"], W)
+        ids = torch.randint(0, z["vocab"], (T,), device=dev)
+        add("scaled_embedding (residual, rows, split)", phase, lambda: mix_ops.scaled_embedding(ids, table, 45.0, True, True), nbytes=T * W * 12)
+        add("bisuzen embedding lookup, widening copy, norm", phase,
+            lambda: mix_ops.residual_dyt(torch.nn.functional.embedding(ids, table).float(), alpha=alpha, w=nw, b=nw, act_dtype=bf),
+            nbytes=T * W * 8, like="scaled_embedding")
+        add("residual_split", phase, lambda: mix_ops.residual_split(x, y1), nbytes=T * W * 14)
+        add("residual_add_norm", phase, lambda: mix_ops.residual_add_norm(x, y1, None, nw, 1.0, 1e-6, bf), nbytes=T * W * 12)
+        add("bisuzen residual_dyt", phase, lambda: mix_ops.residual_dyt(x, y1, None, None, None, 1.0, 1e-6, alpha, nw, nw, bf),
+            nbytes=T * W * 12, like="residual_split, residual_add_norm")
+        sp, wl, x0 = mix_ops.residual_split(x, y1), rand(W, 2 * W), rand(T, W, dtype=torch.float32)
+        add("entry of a pass: f32 product of the split residual (library)", phase, lambda: mix_ops.mm_f32(sp, wl.t(), add=x0),
+            flops=T * W * W * 4, matrix=True, nbytes=(W * W * 4 + T * W * 12) if decode else 0)
+        # attention with distance biases
+        proj = rand(T, H * D + 2 * G * D)
+        kc, vc = (torch.zeros(pages, page, G, D, device=dev, dtype=bf) for _ in range(2))
+        ks = torch.ones(pages, page, G, device=dev)
+        qw, sinks = torch.ones(D, device=dev), torch.zeros(H, device=dev)
+        add("head_norm_store", phase, lambda: mix_ops.head_norm_store(proj, 0, H * D, qw, kc, ks, step, H, G, D, 1e-6),
+            nbytes=T * (H + G) * D * 4)
+        add("bisuzen qk_prep_store (heads divided by their rms)", phase,
+            lambda: mix_ops.rotary_store(proj, 0, H * D, H * D + G * D, None, None, kc, vc, step, H, G, D, D, 0, unit_eps=1e-6),
+            nbytes=T * (H + 2 * G) * D * 4, like="head_norm_store")
+        q = mix_ops.head_norm_store(proj, 0, H * D, qw, kc, ks, step, H, G, D, 1e-6)
+        bias = mix_ops.distance_bias(rand(kz["rel_rows"], H, dtype=torch.float32), kz["rel_far"], window)
+        wide = torch.empty(T, H * D + ff, device=dev, dtype=bf)
+        keys = sum(min(i + 1, window) for n_, c0 in zip(lens_q, ctx) for i in range(c0, c0 + n_))
+
+        def att_work(key_bytes, flops):
+            return dict(nbytes=keys * key_bytes) if decode else dict(flops=keys * flops, matrix=True)
+        add("attention, distance biases, keys as values", phase,
+            lambda: mix_ops.window_pool_attention(q, kc, kc, None, None, None, step, H, G, D, D, window, 0, D ** -0.5, has_sink=False,
+                                                  sinks=sinks, key_scale=ks, dist_bias=bias, out=wide[:, :H * D]),
+            **att_work(G * (D * 2 + 4), H * D * 4))
+        add("bisuzen windowed attention with sinks, same keys", phase,
+            lambda: mix_ops.window_pool_attention(q, kc, vc, None, None, None, step, H, G, D, D, window, 0, D ** -0.5, has_sink=False,
+                                                  sinks=sinks), like="attention, distance biases", **att_work(G * D * 4, H * D * 4))
+        # latent attention
+        nq = H * (D + Dr)
+        lproj = rand(T, nq + R + Dr)
+        lw = torch.ones(R, device=dev)
+        freq = mix_ops.rotary_inv_freq(Dr, 10000.0, dev)
+        lc = torch.zeros(pages, page, R + Dr, device=dev, dtype=bf)
+        q_abs = rand(T, H, R + Dr)
+        add("latent_store", phase, lambda: mix_ops.latent_store(lproj, 0, nq, lw, freq, 1.2, q_abs, lc, step, H, D, Dr, R, Dr, True, 1e-6),
+            nbytes=T * (R + Dr + H * Dr) * 4)
+        Rq = W * 3 // 8
+        pproj, pq, plat = rand(T, Rq + R + Dr), rand(T, nq), rand(H, T, R)
+        pw = torch.ones(Rq, device=dev)
+        add("bokulorn latent_prep and latent_q_finish", phase,
+            lambda: (mix_ops.latent_prep(pproj, 0, Rq, pw, lw, freq, lc, step, Rq, R, Dr, Dr, 1e-6),
+                     mix_ops.latent_q_finish(pq, plat, freq, step, H, D, Dr, R, Dr)),
+            nbytes=T * (Rq + R + Dr + H * (R + Dr)) * 4, like="latent_store")
+        rows_ = lc.unsqueeze(2)
+        qa = q_abs.view(T, H * (R + Dr))
+        add("latent attention, window and sinks", phase,
+            lambda: mix_ops.window_pool_attention(qa, rows_, rows_[..., :R], None, None, None, step, H, 1, R + Dr, R, window, 0,
+                                                  (D + Dr) ** -0.5, has_sink=False, sinks=sinks),
+            **att_work((R + Dr) * 2, H * (2 * R + Dr) * 2))
+        add("bokulorn latent attention, same keys", phase,
+            lambda: mix_ops.window_pool_attention(qa, rows_, rows_[..., :R], None, None, None, step, H, 1, R + Dr, R, window, 0,
+                                                  (D + Dr) ** -0.5, has_sink=False), like="latent attention",
+            **att_work((R + Dr) * 2, H * (2 * R + Dr) * 2))
+        uk, uv = rand(H, D, R), rand(H, R, D)
+        lq = lproj[:, :nq].view(T, H, D + Dr)[:, :, :D].transpose(0, 1)
+        o_lat = rand(T, H, R).transpose(0, 1)
+        mm_work = dict(flops=T * H * D * R * 2, matrix=True, nbytes=H * D * R * 2 if decode else 0)
+        add("latent attention: queries into the latent space (library)", phase,
+            lambda: torch.bmm(lq, uk, out=q_abs[:, :, :R].transpose(0, 1)), **mm_work)
+        add("latent attention: values out of it (library)", phase,
+            lambda: torch.bmm(o_lat, uv, out=wide[:, :H * D].view(T, H, D).transpose(0, 1)), **mm_work)
+        # recurrence
+        N = W
+        rproj = rand(T, 2 * N + 2 * ff)
+        cw, cb = rand(N, taps, dtype=torch.float32), rand(N, dtype=torch.float32)
+        cstate = torch.zeros(B, taps - 1, N, device=dev, dtype=bf)
+        conv_bytes = T * N * 4 + N * taps * 4 + B * (taps - 1) * N * 4
+        add("causal_conv", phase, lambda: mix_ops.causal_conv(rproj[:, N:2 * N], cw, cb, cstate, step), nbytes=conv_bytes)
+        add("feditar causal_conv with silu", phase, lambda: mix_ops.causal_conv(rproj[:, N:2 * N], cw, cb, cstate, step, silu=True),
+            nbytes=conv_bytes, like="causal_conv")
+        n = N // blocks
+        gw, gb = rand(blocks, 2, n, n) * n ** -0.5, torch.zeros(blocks, 2, n, device=dev)
+        rate, state = torch.full((N,), -0.4, device=dev), torch.zeros(B, N, device=dev)
+        u = rand(T, N)
+        lru_bytes = T * N * 6 + blocks * 2 * n * n * 2 + B * N * 8
+        add("gated_linear_recurrence", phase,
+            lambda: mix_ops.gated_linear_recurrence(u, rproj[:, :N], gw, gb, rate, state, step, blocks, out=wide[:, :N]),
+            nbytes=lru_bytes, flops=T * N * n * 4, matrix=True)
+        # the recurrences of the other models at their own state sizes; one launch takes all of a layer's channels
+        Hs = H
+        sproj, decay, S4 = rand(T, 4 * Hs * D), torch.full((Hs,), 0.99, device=dev), torch.zeros(B, Hs, D, D, device=dev)
+        add("bisuzen lightning_attention", phase,
+            lambda: mix_ops.lightning_attention(sproj, 0, Hs * D, 2 * Hs * D, decay, S4, step, Hs, D, D), like="gated_linear_recurrence",
+            flops=T * Hs * D * D * 4, nbytes=B * Hs * D * D * 8 + T * Hs * D * 10)
+        Hx, Dx, Ns, Gx = fz["ssm_heads"], fz["ssm_vdim"], fz["ssm_state"], fz["ssm_groups"]
+        inner = Hx * Dx
+        ux, dt = rand(T, inner + 2 * Gx * Ns), rand(T, Hx)
+        xs, xB, xC = torch.split(ux, [inner, Gx * Ns, Gx * Ns], dim=1)
+        dtb, al, sk = torch.full((Hx,), -3.0, device=dev), torch.zeros(Hx, device=dev), torch.ones(Hx, device=dev)
+        S2 = torch.zeros(B, Hx, Ns, Dx, device=dev)
+        add("feditar gated_scan (state space)", phase,
+            lambda: mix_ops.gated_scan(mix_ops.SCAN_STEP, xC, xB, xs, dt, dtb, al, step, S2, Hx, Gx, Ns, Dx, p2=sk), like="gated_linear_recurrence",
+            flops=T * Hx * Ns * Dx * 4, nbytes=B * Hx * Ns * Dx * 8 + T * (inner * 6 + Gx * Ns * 4))
+        # feed-forward
+        add("glu_act (relu)", phase, lambda: mix_ops.glu_act(rproj[:, 2 * N:], "relu", out=wide[:, N:N + ff]), nbytes=T * ff * 6)
+        zg = rand(T, 2 * ff)
+        add("bisuzen glu_act (tanh gelu)", phase, lambda: mix_ops.glu_act(zg, "gelu_tanh"), nbytes=T * ff * 6, like="glu_act (relu)")
+    return rows
+
+
+def gokolix_leg(sizes, batch, prompt_len, new_tokens, engine_only=False):
+    dev = torch.device("cuda:0")
+    torch.cuda.set_device(dev)
+    out = {"metric": "mixers: Gokolix beside Bisuzen at equal size", "dtype": "bf16", "data": "synthetic, random weights",
+           "batch": batch, "prompt_len": prompt_len, "new_tokens": new_tokens, "sizes": []}
+    for name in sizes:
+        z, kz, sz, fz = MIXER_SIZES[name], GOKOLIX_SIZES[name], BISUZEN_SIZES[name], FEDITAR_SIZES[name]
+        rec = {"size": name, **z, **kz}
+        cache_tokens = batch * 256 * (-(-(prompt_len + new_tokens) // 256))
+        kw = dict(kvcache_block_size=256, max_cache_tokens=cache_tokens)
+        rec["gokolix"] = _engine_rates(_gokolix_config(z, kz), batch, prompt_len, new_tokens, **kw)
+        rec["gokolix_graph"] = _engine_rates(_gokolix_config(z, kz), batch, prompt_len, new_tokens, enforce_eager=False, **kw)
+        if not engine_only:
+            rec["bisuzen"] = _engine_rates(_bisuzen_config(z, sz), batch, prompt_len, new_tokens, **kw)
+            rec["bisuzen_graph"] = _engine_rates(_bisuzen_config(z, sz), batch, prompt_len, new_tokens, enforce_eager=False, **kw)
+            rec["kernels"] = _gokolix_kernel_table(z, kz, fz, dev, batch, prompt_len)
+        out["sizes"].append(rec)
+    print(json.dumps(out), flush=True)
+
+
 def mixers_leg(sizes, batch, prompt_len, new_tokens):
     dev = torch.device("cuda:0")
     torch.cuda.set_device(dev)
@@ -1532,16 +1735,19 @@ def main():
                          "(proves launcher, rendezvous, graph and JSON path; not a measurement)")
     ap.add_argument("--mixers", default="", help="comma list of sizes (2k, 4k): instead of the default workload, "
                     "run the Kagalorn design beside Qwen3 at equal size and time its kernels one by one")
-    ap.add_argument("--mixers-design", default="kagalorn", choices=("kagalorn", "bokulorn", "givozen", "bisuzen", "feditar"),
+    ap.add_argument("--mixers-design", default="kagalorn", choices=("kagalorn", "bokulorn", "givozen", "bisuzen", "feditar", "gokolix"),
                     help="with --mixers: kagalorn (beside Qwen3), bokulorn (beside Kagalorn, its closest relative) or "
                          "givozen (beside Bokulorn, its closest relative) or bisuzen (beside Givozen, its closest relative) or "
-                         "feditar (beside Bisuzen, its closest relative)")
+                         "feditar or gokolix (beside Bisuzen, their closest relative)")
     ap.add_argument("--mixers-engine-only", action="store_true",
-                    help="with --mixers-design bisuzen or feditar: only that design's engine runs (eager and from graphs), for a profiler")
+                    help="with --mixers-design bisuzen, feditar or gokolix: only that design's engine runs (eager and from graphs), for a profiler")
     ap.add_argument("--mixers-batch", type=int, default=16)
     ap.add_argument("--mixers-prompt", type=int, default=1024)
     ap.add_argument("--mixers-new", type=int, default=17)
     args = ap.parse_args()
+    if args.mixers and args.mixers_design == "gokolix":
+        return gokolix_leg([x for x in args.mixers.split(",") if x], args.mixers_batch, args.mixers_prompt, args.mixers_new,
+                           args.mixers_engine_only)
     if args.mixers and args.mixers_design == "feditar":
         return feditar_leg([x for x in args.mixers.split(",") if x], args.mixers_batch, args.mixers_prompt, args.mixers_new,
                            args.mixers_engine_only)
