@@ -6,13 +6,16 @@
 // query does not see (outside its window, a block not yet wholly before it, the future) is masked.
 //
 // Everything is computed transposed so that no operand changes layout between the two products:
-//   S^T = K Q^T   v_mfma_f32_16x16x32_bf16 (one 16x16x16 step more when D is an odd multiple of 16), A = 16 keys x 32
-//                 of D read straight from the cache rows with 16-byte loads, B = the wave's Q fragments (registers,
-//                 loaded once); a lane ends up with 4 keys of ONE query, so the softmax statistics of a query live
-//                 in 4 lanes (two shuffles) and
+//   S^T = K Q^T   v_mfma_f32_16x16x32_bf16, A = 16 keys x 32 of D read straight from the cache rows with 16-byte loads, B = the
+//                 wave's Q fragments (registers, loaded once); a lane ends up with 4 keys of ONE query, so the softmax
+//                 statistics of a query live in 4 lanes (two shuffles) and
 //   O^T += V^T P^T  takes the probabilities of two 16-key blocks as its B operand exactly as they lie (keys x
-//                 queries), with A = V^T read as two 8-byte runs of keys from the 64-entry V tile that the four
-//                 waves stage TRANSPOSED in LDS together.
+//                 queries), with A = V^T from transposing LDS reads of the 64-entry V tile that the four waves stage
+//                 together, rows as they are.
+// Fragment counts are compile-time bounds and nothing in the tile loop branches on the head sizes: a step past the end of D reads
+// the last entries of the row again against zeros in Q, a block past Dv reads the last block of V and is not stored. (With a
+// branch around every load and its MFMA the loads could not be issued together, and the kernel ran at one memory latency per
+// MFMA.)
 // The sink is the initial state of the running softmax: maximum 0 (or the head's learned number), sum 1.
 // Extended form: a tile's key factors (norms kept beside unnormed keys) and the heads' distance biases sit in LDS; a score becomes
 // product * scale * factor + bias before the softmax.
@@ -20,9 +23,12 @@
 
 namespace lvmix {
 
-typedef __attribute__((ext_vector_type(4))) short bf16x4_t;
+typedef __attribute__((ext_vector_type(4))) __bf16 bf16x4v_t;
+typedef __attribute__((address_space(3))) __bf16 lds_bf16;
+typedef __attribute__((address_space(3))) bf16x4v_t lds_bf16x4;
 typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8_t;
 typedef __attribute__((ext_vector_type(4))) float f32x4_t;
+typedef __attribute__((ext_vector_type(4))) uint32_t u32x4_t;
 
 struct WindowMfmaParams {
   const uint16_t *q, *k_cache, *v_cache, *kp, *vp, *gate;
@@ -51,8 +57,9 @@ enum ScoreForm { kPlain = 0, kCapped = 1, kExtended = 2 };
 
 constexpr int kTileQ = 16;
 constexpr int kTileK = 64;
-constexpr int kMaxK32 = 8;     // D <= 256: 32-wide steps over D (template K32: 4 up to D = 128), plus one 16-wide when D % 32 == 16
-constexpr int kLdk = kTileK + 4; // row stride (in keys) of the transposed V tile: rows stay 8-byte aligned
+constexpr int kMaxK32 = 8;     // D <= 256: 32-wide steps over D (template K32: 2, 4 or 8)
+// Row stride of the V tile: an odd multiple of 16 entries, so that the 16 rows a transposed read touches lie in all banks.
+__host__ __device__ constexpr int v_row(int Dv) { return Dv % 32 == 0 ? Dv + 16 : Dv; }
 constexpr int kMaxDvb = 16;    // Dv <= 256
 constexpr int kBiasLds = 1024; // distance biases of a head up to this many are copied to LDS (longer tables are read from memory)
 constexpr int kBtCache = 2048; // page ids of a sequence kept in LDS (longer sequences look them up in memory)
@@ -80,8 +87,8 @@ __device__ __forceinline__ float fast_tanh(float x) { return 1.0f - 2.0f * __bui
 // ahead the kernel fell from two waves a SIMD to one and ran 1.7x slower; K32 and DVB size the fragment arrays for the
 // head sizes at hand for the same reason.
 template <bool AHEAD, int K32, int DVB, int FORM>
-__global__ __launch_bounds__(256, (AHEAD || DVB > 8) ? 1 : 4) void window_pool_mfma_kernel(WindowMfmaParams p) {
-  extern __shared__ uint16_t vs[];                      // V^T tile [Dv][kLdk]
+__global__ __launch_bounds__(256, AHEAD ? 1 : (DVB > 8 ? 2 : (DVB > 4 ? 3 : 4))) void window_pool_mfma_kernel(WindowMfmaParams p) {
+  extern __shared__ __attribute__((aligned(16))) uint16_t vs[];             // V tile [kTileK][ldv]
   const int wave = threadIdx.x / kWave, lane = threadIdx.x % kWave;
   const int ln = lane & 15, lg = lane >> 4;
   const int b = blockIdx.z;
@@ -102,8 +109,9 @@ __global__ __launch_bounds__(256, (AHEAD || DVB > 8) ? 1 : 4) void window_pool_m
   const bool active = hloc < rep;
   const int h = g * rep + min(hloc, rep - 1);
   const int D = p.D, Dv = p.Dv, page = p.page, P = p.P, W = p.window;
-  const int nk32 = D / 32, ndvb = Dv / 16;
-  const bool tail16 = (D & 16) != 0;
+  const int ndvb = Dv / 16, ldv = v_row(Dv);
+  // transposed reads: of every 4 keys x 16 columns, lane 4 q + r of 16 names key q, columns 4r .. 4r + 3, and gets column 4 q + r of all four
+  const lds_bf16* vt0 = (const lds_bf16*)vs + (4 * lg + (ln >> 2)) * ldv + 4 * (ln & 3);
   const int64_t GD = static_cast<int64_t>(p.G) * D, GDv = static_cast<int64_t>(p.G) * Dv;
   const int32_t* bt_global = p.block_tables + static_cast<int64_t>(b) * p.bt_stride;
   // the sequence's page ids up to the last query's page, once, so that no row address waits for a second trip to memory
@@ -116,7 +124,7 @@ __global__ __launch_bounds__(256, (AHEAD || DVB > 8) ? 1 : 4) void window_pool_m
   }
   auto bt = [&](int idx) { return bt_cached ? bt_lds[idx] : bt_global[idx]; };
   // kExtended: the tile's key factors and the distance biases of the workgroup's heads, behind the V tile
-  float* ks_lds = reinterpret_cast<float*>(vs + Dv * kLdk);                // [kTileK]
+  float* ks_lds = reinterpret_cast<float*>(vs + kTileK * ldv);             // [kTileK]
   float* bias_lds = ks_lds + kTileK;                                       // [4][bias_len]
   const float* bias_h = nullptr;
   bool bias_cached = false;
@@ -124,20 +132,20 @@ __global__ __launch_bounds__(256, (AHEAD || DVB > 8) ? 1 : 4) void window_pool_m
     if (p.dist_bias != nullptr) {
       bias_cached = p.bias_len <= kBiasLds;
       bias_h = p.dist_bias + static_cast<int64_t>(h) * p.bias_len;
-      if (bias_cached)
-        for (int x = lane; x < p.bias_len; x += kWave) bias_lds[wave * p.bias_len + x] = bias_h[x];   // read by this wave alone
     }
     if (p.key_scale == nullptr && threadIdx.x < kTileK) ks_lds[threadIdx.x] = 1.0f;                 // read behind the first barrier
   }
 
   bf16x8_t qf[K32];
-  bf16x4_t qtail = bf16x4_t{0, 0, 0, 0};
+  int koff[K32];                                        // this lane's entries of a key or query row in step kk
   {
     const uint16_t* qrow = p.q + (t * p.H + h) * D;
 #pragma unroll
-    for (int kk = 0; kk < K32; ++kk)
-      if (kk < nk32) qf[kk] = *reinterpret_cast<const bf16x8_t*>(qrow + 32 * kk + 8 * lg);
-    if (tail16) qtail = *reinterpret_cast<const bf16x4_t*>(qrow + 32 * nk32 + 4 * lg);
+    for (int kk = 0; kk < K32; ++kk) {
+      koff[kk] = min(32 * kk + 8 * lg, D - 8);
+      qf[kk] = *reinterpret_cast<const bf16x8_t*>(qrow + koff[kk]);
+      if (32 * kk + 8 * lg >= D) qf[kk] = __builtin_bit_cast(bf16x8_t, u32x4_t{0, 0, 0, 0});
+    }
   }
   f32x4_t acc_o[DVB];
 #pragma unroll
@@ -155,67 +163,44 @@ __global__ __launch_bounds__(256, (AHEAD || DVB > 8) ? 1 : 4) void window_pool_m
   const int npt = (nbmax + kTileK - 1) / kTileK;
   const int ntt = (i1 + 1 - jlo + kTileK - 1) / kTileK;
   const int ntiles = npt + ntt;
-  const int nseg = Dv / 4;                                                // 8-byte segments of a row
+  const int nseg = Dv / 8;                                                // 16-byte segments of a row
 
-  auto entry_rows = [&](int tile, int e, const uint16_t*& kr_, const uint16_t*& vr_) {
-    if (tile < npt && P == 0) {
-      const int ec = min(e, nbmax - 1);
-      const int pj = fdiv(ec, page, p.m_page);
-      const int64_t slot = static_cast<int64_t>(bt(pj)) * page + (ec - pj * page);
-      kr_ = p.k_cache + slot * p.k_ld + g * D;
-      vr_ = p.v_cache + slot * p.v_ld + g * Dv;
-    } else if (tile < npt) {
-      const int ec = min(e, nbmax - 1);
-      const int pj = fdiv(ec * P + P - 1, page, p.m_page);
-      const int64_t slot = static_cast<int64_t>(bt(pj)) * p.PP + (ec - fdiv(page * pj, P, p.m_P));
-      kr_ = p.kp + slot * GD + g * D;
-      vr_ = p.vp + slot * GDv + g * Dv;
-    } else {
-      const int ec = min(e, i1);
-      const int pj = fdiv(ec, page, p.m_page);
-      const int64_t slot = static_cast<int64_t>(bt(pj)) * page + (ec - pj * page);
-      kr_ = p.k_cache + slot * p.k_ld + g * D;
-      vr_ = p.v_cache + slot * p.v_ld + g * Dv;
-    }
-  };
   auto tile_start = [&](int tile) { return tile < npt ? tile * kTileK : jlo + (tile - npt) * kTileK; };
 
-  // V rows of a tile: consecutive threads take consecutive 8-byte segments of a row (whole cache lines per load
-  // instruction). AHEAD: all of a thread's loads are issued together, one tile ahead of their use, and wait in registers.
-  // kExtended: the key factor of entry e of the token tiles or of the kept first tokens
-  auto key_factor = [&](int tile, int e) {
+  // Cache row of entry `lane` of a tile: every wave finds its 64 rows once, a lane each, and hands them round by shuffles.
+  auto tile_slot = [&](int tile) {
+    const int e = tile_start(tile) + lane;
+    if (tile < npt && P > 0) {
+      const int ec = min(e, nbmax - 1);
+      const int pj = fdiv(ec * P + P - 1, page, p.m_page);
+      return bt(pj) * p.PP + (ec - fdiv(page * pj, P, p.m_P));
+    }
     const int ec = min(e, tile < npt ? nbmax - 1 : i1);
     const int pj = fdiv(ec, page, p.m_page);
-    return p.key_scale[(static_cast<int64_t>(bt(pj)) * page + (ec - pj * page)) * p.G + g];
+    return bt(pj) * page + (ec - pj * page);
   };
+  // V rows of a tile: consecutive threads take consecutive 16-byte segments of a row (whole cache lines per load instruction),
+  // all of a thread's loads are issued together. AHEAD: one tile ahead of their use, and they wait in registers.
+  constexpr int NV = DVB / 2;
   const bool keyed = FORM == kExtended && p.key_scale != nullptr && threadIdx.x < kTileK;
   float ksreg = 1.0f;
-  uint2 vreg[AHEAD ? DVB : 1];
+  u32x4_t vreg[NV];
   const uint16_t* knext[4];
-  auto prefetch = [&](int tile) {
-    const int e0 = tile_start(tile);
+  auto fetch_rows = [&](int tile) {
+    const int slot = tile_slot(tile);
+    const bool pooled = tile < npt && P > 0;
+    const uint16_t* kbase = (pooled ? p.kp : p.k_cache) + g * D;
+    const uint16_t* vbase = (pooled ? p.vp : p.v_cache) + g * Dv;
+    const int64_t kld = pooled ? GD : p.k_ld, vld = pooled ? GDv : p.v_ld;
 #pragma unroll
-    for (int x = 0; x < (AHEAD ? DVB : 0); ++x) {
-      const int c = threadIdx.x + 256 * x;
-      if (c < kTileK * nseg) {
-        const int row = fdiv(c, nseg, p.m_nseg), seg = c - row * nseg;
-        const uint16_t *kr_, *vr_;
-        entry_rows(tile, e0 + row, kr_, vr_);
-        vreg[x] = *reinterpret_cast<const uint2*>(vr_ + seg * 4);
-      }
+    for (int x = 0; x < NV; ++x) {
+      const int c = min(static_cast<int>(threadIdx.x) + 256 * x, kTileK * nseg - 1);
+      const int row = fdiv(c, nseg, p.m_nseg), seg = c - row * nseg;
+      vreg[x] = *reinterpret_cast<const u32x4_t*>(vbase + __shfl(slot, row, kWave) * vld + seg * 8);
     }
 #pragma unroll
-    for (int kb = 0; kb < 4; ++kb) {
-      const uint16_t* unused;
-      entry_rows(tile, e0 + kb * 16 + ln, knext[kb], unused);
-    }
-    if (keyed) ksreg = key_factor(tile, e0 + threadIdx.x);
-  };
-  auto store_v = [&](uint16_t* dst, uint2 v4) {
-    dst[0] = static_cast<uint16_t>(v4.x & 0xffffu);
-    dst[kLdk] = static_cast<uint16_t>(v4.x >> 16);
-    dst[2 * kLdk] = static_cast<uint16_t>(v4.y & 0xffffu);
-    dst[3 * kLdk] = static_cast<uint16_t>(v4.y >> 16);
+    for (int kb = 0; kb < 4; ++kb) knext[kb] = kbase + __shfl(slot, kb * 16 + ln, kWave) * kld;
+    if (keyed) ksreg = p.key_scale[static_cast<int64_t>(slot) * p.G + g];    // the first wave: lane = entry
   };
   // Only LDS traffic meets at the barriers of the tile loop. The fetch-ahead variant waits for that alone, so that the
   // vector loads of the next tile stay in flight across them (a full __syncthreads would drain them every tile).
@@ -224,57 +209,42 @@ __global__ __launch_bounds__(256, (AHEAD || DVB > 8) ? 1 : 4) void window_pool_m
     else __syncthreads();
   };
   bf16x8_t kdata[AHEAD ? 4 : 1][K32];
-  bf16x4_t ktail[4];
   auto fetch_k = [&]() {                                                    // the K fragments of the tile knext points to
 #pragma unroll
     for (int kb = 0; kb < (AHEAD ? 4 : 0); ++kb) {
 #pragma unroll
-      for (int kk = 0; kk < K32; ++kk)
-        if (kk < nk32) kdata[kb][kk] = *reinterpret_cast<const bf16x8_t*>(knext[kb] + 32 * kk + 8 * lg);
-      if (tail16) ktail[kb] = *reinterpret_cast<const bf16x4_t*>(knext[kb] + 32 * nk32 + 4 * lg);
+      for (int kk = 0; kk < K32; ++kk) kdata[kb][kk] = *reinterpret_cast<const bf16x8_t*>(knext[kb] + koff[kk]);
     }
   };
   // a split takes a contiguous share of the tiles
   const int per_split = p.nsplit > 1 ? (ntiles + p.nsplit - 1) / p.nsplit : ntiles;
   const int t_begin = split * per_split, t_end = min(ntiles, t_begin + per_split);
   if (AHEAD && t_begin < t_end) {
-    prefetch(t_begin);
+    fetch_rows(t_begin);
     if (active) fetch_k();
   }
+  if (bias_cached)                                                         // behind the first tile's requests; read by this wave alone
+    for (int x = lane; x < p.bias_len; x += kWave) bias_lds[wave * p.bias_len + x] = bias_h[x];
   for (int tile = t_begin; tile < t_end; ++tile) {
     const int phase = tile < npt ? 0 : 1;
     const int e0 = tile_start(tile);
     const int e_end = phase == 0 ? nbmax : i1 + 1;
     const uint16_t* kcur[4];
     tile_barrier();                                                         // the previous tile's V reads are done
-    if constexpr (AHEAD) {
+    if constexpr (!AHEAD) fetch_rows(tile);
 #pragma unroll
-      for (int x = 0; x < DVB; ++x) {
-        const int c = threadIdx.x + 256 * x;
-        if (c < kTileK * nseg) {
-          const int row = fdiv(c, nseg, p.m_nseg), seg = c - row * nseg;
-          store_v(vs + (seg * 4) * kLdk + row, vreg[x]);
-        }
-      }
-#pragma unroll
-      for (int kb = 0; kb < 4; ++kb) kcur[kb] = knext[kb];
-      if (keyed) ks_lds[threadIdx.x] = ksreg;
-    } else {
-      if (keyed) ks_lds[threadIdx.x] = key_factor(tile, e0 + threadIdx.x);
-      for (int c = threadIdx.x; c < kTileK * nseg; c += blockDim.x) {
+    for (int x = 0; x < NV; ++x) {
+      const int c = threadIdx.x + 256 * x;
+      if (c < kTileK * nseg) {
         const int row = fdiv(c, nseg, p.m_nseg), seg = c - row * nseg;
-        const uint16_t *kr_, *vr_;
-        entry_rows(tile, e0 + row, kr_, vr_);
-        store_v(vs + (seg * 4) * kLdk + row, *reinterpret_cast<const uint2*>(vr_ + seg * 4));
-      }
-#pragma unroll
-      for (int kb = 0; kb < 4; ++kb) {
-        const uint16_t* unused;
-        entry_rows(tile, e0 + kb * 16 + ln, kcur[kb], unused);
+        *reinterpret_cast<u32x4_t*>(vs + row * ldv + seg * 8) = vreg[x];
       }
     }
+#pragma unroll
+    for (int kb = 0; kb < 4; ++kb) kcur[kb] = knext[kb];
+    if (keyed) ks_lds[threadIdx.x] = ksreg;
     tile_barrier();
-    if (AHEAD && tile + 1 < t_end) prefetch(tile + 1);
+    if (AHEAD && tile + 1 < t_end) fetch_rows(tile + 1);
     if (!active) continue;
     {
       float s[4][4];
@@ -284,12 +254,8 @@ __global__ __launch_bounds__(256, (AHEAD || DVB > 8) ? 1 : 4) void window_pool_m
         f32x4_t acc = f32x4_t{0.0f, 0.0f, 0.0f, 0.0f};
 #pragma unroll
         for (int kk = 0; kk < K32; ++kk)
-          if (kk < nk32)
-            acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-                AHEAD ? kdata[AHEAD ? kb : 0][kk] : *reinterpret_cast<const bf16x8_t*>(krow + 32 * kk + 8 * lg), qf[kk], acc, 0, 0, 0);
-        if (tail16)
-          acc = __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(
-              AHEAD ? ktail[kb] : *reinterpret_cast<const bf16x4_t*>(krow + 32 * nk32 + 4 * lg), qtail, acc, 0, 0, 0);
+          acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+              AHEAD ? kdata[AHEAD ? kb : 0][kk] : *reinterpret_cast<const bf16x8_t*>(krow + koff[kk]), qf[kk], acc, 0, 0, 0);
         float4 ks = float4{1.0f, 1.0f, 1.0f, 1.0f};
         if constexpr (FORM == kExtended) ks = *reinterpret_cast<const float4*>(ks_lds + kb * 16 + 4 * lg);
 #pragma unroll
@@ -339,19 +305,15 @@ __global__ __launch_bounds__(256, (AHEAD || DVB > 8) ? 1 : 4) void window_pool_m
       l = l * corr + rs;
       m = nm;
 #pragma unroll
-      for (int d = 0; d < DVB; ++d)
-        if (d < ndvb) acc_o[d] *= corr;
+      for (int d = 0; d < DVB; ++d) acc_o[d] *= corr;
 #pragma unroll
-      for (int c = 0; c < 2; ++c) {
-        const uint16_t* vt = vs + ln * kLdk + c * 32 + 4 * lg;              // value column ln: keys 4lg.. of blocks 2c, 2c+1
+      for (int c = 0; c < 2; ++c) {                                         // key blocks 2c and 2c + 1
 #pragma unroll
         for (int d = 0; d < DVB; ++d) {
-          if (d < ndvb) {
-            const uint2 lo = *reinterpret_cast<const uint2*>(vt + 16 * d * kLdk);
-            const uint2 hi = *reinterpret_cast<const uint2*>(vt + 16 * d * kLdk + 16);
-            const uint4 both = uint4{lo.x, lo.y, hi.x, hi.y};
-            acc_o[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, both), pb[c], acc_o[d], 0, 0, 0);
-          }
+          const lds_bf16* vt = vt0 + 32 * c * ldv + 16 * min(d, ndvb - 1);
+          const bf16x4v_t lo = __builtin_amdgcn_ds_read_tr16_b64_v4bf16((lds_bf16x4*)vt);
+          const bf16x4v_t hi = __builtin_amdgcn_ds_read_tr16_b64_v4bf16((lds_bf16x4*)(vt + 16 * ldv));
+          acc_o[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7), pb[c], acc_o[d], 0, 0, 0);
         }
       }
     }
@@ -398,15 +360,22 @@ __global__ __launch_bounds__(256) void window_pool_merge_kernel(const float* __r
   const int64_t t = item / H;
   const int h = static_cast<int>(item - t * H);
   const float* w = ws + item * nsplit * (Dv + 4);
-  float mm = sinks != nullptr ? sinks[h] : m0;
-  for (int s = 0; s < nsplit; ++s) mm = fmaxf(mm, w[s * (Dv + 4) + Dv]);
-  float ll = 0.0f;
-  for (int s = 0; s < nsplit; ++s) ll += w[s * (Dv + 4) + Dv + 1] * expf(w[s * (Dv + 4) + Dv] - mm);
+  // lane s holds split s (at most kWave of them): its maximum and sum, then the factor that brings it to the common maximum
+  const float m0h = sinks != nullptr ? sinks[h] : m0;
+  const bool in = lane < nsplit;
+  const float ms = in ? w[lane * (Dv + 4) + Dv] : -INFINITY, ls = in ? w[lane * (Dv + 4) + Dv + 1] : 0.0f;
+  const float mm = fmaxf(m0h, wave_max(ms));
+  const float f = in ? expf(ms - mm) : 0.0f;
+  const float ll = wave_sum(ls * f);
   const float inv = ll > 0.0f ? 1.0f / ll : 0.0f;
-  for (int dv = lane; dv < Dv; dv += kWave) {
+  for (int dv0 = 0; dv0 < Dv; dv0 += kWave) {                               // the same trip count for every lane: the factors are shuffled
+    const int dv = dv0 + lane;
+    const float* col = w + min(dv, Dv - 1);
     float acc = 0.0f;
-    for (int s = 0; s < nsplit; ++s) acc += w[s * (Dv + 4) + dv] * expf(w[s * (Dv + 4) + Dv] - mm);
+#pragma unroll 4
+    for (int s = 0; s < nsplit; ++s) acc += col[s * (Dv + 4)] * __shfl(f, s, kWave);
     float val = acc * inv;
+    if (dv >= Dv) continue;
     if (gate != nullptr)
       val *= sigmoidf_(__builtin_bit_cast(float, static_cast<uint32_t>(gate[t * ld_gate + static_cast<int64_t>(h) * gate_dv +
                                                                             (gate_dv > 1 ? dv : 0)]) << 16));
@@ -455,8 +424,8 @@ extern "C" int lv_masked_attn_mfma(const void* q, const void* k_cache, const voi
   if (gate != nullptr && ld_gate < static_cast<int64_t>(H) * gate_dv) return fail(-1, "lv_window_pool_attn_mfma: gate stride");
   if (k_ld <= 0) k_ld = static_cast<int64_t>(G) * D;
   if (v_ld <= 0) v_ld = static_cast<int64_t>(G) * Dv;
-  if (k_ld < static_cast<int64_t>(G) * D || v_ld < static_cast<int64_t>(G) * Dv || k_ld % 8 != 0 || v_ld % 4 != 0 ||
-      (reinterpret_cast<uintptr_t>(k_cache) & 15) != 0 || (reinterpret_cast<uintptr_t>(v_cache) & 7) != 0)
+  if (k_ld < static_cast<int64_t>(G) * D || v_ld < static_cast<int64_t>(G) * Dv || k_ld % 8 != 0 || v_ld % 8 != 0 ||
+      (reinterpret_cast<uintptr_t>(k_cache) & 15) != 0 || (reinterpret_cast<uintptr_t>(v_cache) & 15) != 0)
     return fail(-1, "lv_window_pool_attn_mfma: row strides or alignment of the caches");
   const bool extended = extras != nullptr && (extras->key_scale != nullptr || extras->dist_bias != nullptr);
   if (extended && (P > 0 || softcap > 0.0f || (extras->dist_bias != nullptr && extras->bias_len <= 0)))
@@ -471,20 +440,21 @@ extern "C" int lv_masked_attn_mfma(const void* q, const void* k_cache, const voi
                      static_cast<const uint16_t*>(vp), static_cast<const uint16_t*>(gate), ld_gate, gate_dv,
                      static_cast<uint16_t*>(out), cu_q, ctx_lens, block_tables, bt_stride, H, G, D, Dv, page, window, P,
                      P > 0 ? (page + P - 1) / P : 0, ngroups, scale, has_sink ? 1.0f : 0.0f,
-                     magic(page), magic(P > 0 ? P : 1), magic(Dv / 4), nsplit > 1 ? nsplit : 1, static_cast<float*>(workspace),
+                     magic(page), magic(P > 0 ? P : 1), magic(Dv / 8), nsplit > 1 ? nsplit : 1, static_cast<float*>(workspace),
                      k_ld, v_ld, m0, keep_first, chunk, static_cast<const float*>(sinks), softcap > 0.0f ? scale / softcap : 0.0f,
                      softcap, extended ? static_cast<const float*>(extras->key_scale) : nullptr,
                      extended ? static_cast<const float*>(extras->dist_bias) : nullptr, extended ? extras->bias_len : 0, out_ld};
-  if (nsplit > 1 && (max_new_tokens > kTileQ || workspace == nullptr || T <= 0))
+  if (nsplit > 1 && (max_new_tokens > kTileQ || workspace == nullptr || T <= 0 || nsplit > kWave))
     return fail(-1, "lv_window_pool_attn_mfma: key splits need one query tile per sequence and a workspace");
-  size_t shm = static_cast<size_t>(Dv) * kLdk * sizeof(uint16_t);
+  size_t shm = static_cast<size_t>(kTileK) * v_row(Dv) * sizeof(uint16_t);
   if (extended) shm += sizeof(float) * (kTileK + (p.dist_bias != nullptr && p.bias_len <= kBiasLds ? 4 * static_cast<size_t>(p.bias_len) : 0));
   dim3 grid(nsplit > 1 ? nsplit : (max_new_tokens + kTileQ - 1) / kTileQ, G * ngroups, B), block(256);
   hipStream_t st = as_stream(stream);
-  const bool small = D <= 128 && Dv <= 128;
+  const bool tiny = D <= 64 && Dv <= 64, small = D <= 128 && Dv <= 128;
 #define LVMIX_ATT_FORM(AHEAD, FORM)                                                               \
   do {                                                                                            \
-    if (small) window_pool_mfma_kernel<AHEAD, 4, 8, FORM><<<grid, block, shm, st>>>(p);           \
+    if (tiny) window_pool_mfma_kernel<AHEAD, 2, 4, FORM><<<grid, block, shm, st>>>(p);            \
+    else if (small) window_pool_mfma_kernel<AHEAD, 4, 8, FORM><<<grid, block, shm, st>>>(p);      \
     else window_pool_mfma_kernel<AHEAD, kMaxK32, kMaxDvb, FORM><<<grid, block, shm, st>>>(p);     \
   } while (0)
 #define LVMIX_ATT(AHEAD)                                     \

@@ -437,8 +437,8 @@ def window_pool_attention(q, k_cache, v_cache, kp, vp, gate, step, H, G, D, Dv, 
         lib = _mixlib.load()
         extras = _mixlib.AttnExtras(_p(key_scale), _p(dist_bias), dist_bias.size(1) if dist_bias is not None else 0, out.stride(0))
         if (WINDOW_ATTN_KERNEL == "auto" and q.dtype == torch.bfloat16 and D % 16 == 0 and Dv % 16 == 0
-                and D <= 256 and Dv <= 256 and k_ld % 8 == 0 and v_ld % 4 == 0 and k_cache.data_ptr() % 16 == 0
-                and v_cache.data_ptr() % 8 == 0):
+                and D <= 256 and Dv <= 256 and k_ld % 8 == 0 and v_ld % 8 == 0 and k_cache.data_ptr() % 16 == 0
+                and v_cache.data_ptr() % 16 == 0):
             # decode-shaped steps put one workgroup per (sequence, kv head) on the chip: cut each sequence's key
             # tiles over enough workgroups to fill it (partials merged by a second kernel)
             nsplit, ws = 1, None
