@@ -127,11 +127,14 @@ __global__ __launch_bounds__(256, AHEAD ? 1 : (DVB > 8 ? 2 : (DVB > 4 ? 3 : 4)))
   float* ks_lds = reinterpret_cast<float*>(vs + kTileK * ldv);             // [kTileK]
   float* bias_lds = ks_lds + kTileK;                                       // [4][bias_len]
   const float* bias_h = nullptr;
+  float bias_reg[4] = {0.0f, 0.0f, 0.0f, 0.0f};
   bool bias_cached = false;
   if constexpr (FORM == kExtended) {
     if (p.dist_bias != nullptr) {
       bias_cached = p.bias_len <= kBiasLds;
       bias_h = p.dist_bias + static_cast<int64_t>(h) * p.bias_len;
+#pragma unroll
+      for (int x = 0; x < 4; ++x) bias_reg[x] = bias_h[min(lane + x * kWave, p.bias_len - 1)];     // stored behind the first tile's requests
     }
     if (p.key_scale == nullptr && threadIdx.x < kTileK) ks_lds[threadIdx.x] = 1.0f;                 // read behind the first barrier
   }
@@ -223,8 +226,12 @@ __global__ __launch_bounds__(256, AHEAD ? 1 : (DVB > 8 ? 2 : (DVB > 4 ? 3 : 4)))
     fetch_rows(t_begin);
     if (active) fetch_k();
   }
-  if (bias_cached)                                                         // behind the first tile's requests; read by this wave alone
-    for (int x = lane; x < p.bias_len; x += kWave) bias_lds[wave * p.bias_len + x] = bias_h[x];
+  if (bias_cached) {                                                       // read by this wave alone
+#pragma unroll
+    for (int x = 0; x < 4; ++x)
+      if (lane + x * kWave < p.bias_len) bias_lds[wave * p.bias_len + lane + x * kWave] = bias_reg[x];
+    for (int x = lane + 4 * kWave; x < p.bias_len; x += kWave) bias_lds[wave * p.bias_len + x] = bias_h[x];
+  }
   for (int tile = t_begin; tile < t_end; ++tile) {
     const int phase = tile < npt ? 0 : 1;
     const int e0 = tile_start(tile);
@@ -247,39 +254,55 @@ __global__ __launch_bounds__(256, AHEAD ? 1 : (DVB > 8 ? 2 : (DVB > 4 ? 3 : 4)))
     if (AHEAD && tile + 1 < t_end) fetch_rows(tile + 1);
     if (!active) continue;
     {
-      float s[4][4];
+      f32x4_t s[4];
 #pragma unroll
       for (int kb = 0; kb < 4; ++kb) {
         const uint16_t* krow = kcur[kb];
-        f32x4_t acc = f32x4_t{0.0f, 0.0f, 0.0f, 0.0f};
+        s[kb] = f32x4_t{0.0f, 0.0f, 0.0f, 0.0f};
 #pragma unroll
         for (int kk = 0; kk < K32; ++kk)
-          acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-              AHEAD ? kdata[AHEAD ? kb : 0][kk] : *reinterpret_cast<const bf16x8_t*>(krow + koff[kk]), qf[kk], acc, 0, 0, 0);
-        float4 ks = float4{1.0f, 1.0f, 1.0f, 1.0f};
-        if constexpr (FORM == kExtended) ks = *reinterpret_cast<const float4*>(ks_lds + kb * 16 + 4 * lg);
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          const int ke = e0 + kb * 16 + 4 * lg + i;                         // the key of result row 4*lg + i
-          bool vis = ke < e_end;
-          if (phase == 0) vis = vis && (P == 0 || ke * P + P - 1 <= pos - W);
-          else vis = vis && ke <= pos && ((chunk > 0 ? ke >= cstart : pos - ke < W) || ke < keep);
-          float sc;
-          if constexpr (FORM == kCapped) {
-            sc = p.cap * fast_tanh(acc[i] * p.cap_in);
-          } else if constexpr (FORM == kExtended) {
-            sc = acc[i] * (p.scale * (i == 0 ? ks.x : (i == 1 ? ks.y : (i == 2 ? ks.z : ks.w))));
-            if (bias_h != nullptr) {
-              const int dist = min(max(pos - ke, 0), p.bias_len - 1);
-              sc += bias_cached ? bias_lds[wave * p.bias_len + dist] : bias_h[dist];
-            }
-          } else {
-            sc = acc[i] * p.scale;
-          }
-          s[kb][i] = vis ? sc : -INFINITY;
-        }
+          s[kb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+              AHEAD ? kdata[AHEAD ? kb : 0][kk] : *reinterpret_cast<const bf16x8_t*>(krow + koff[kk]), qf[kk], s[kb], 0, 0, 0);
       }
       if (AHEAD && tile + 1 < t_end) fetch_k();                            // in flight across the softmax, PV and the barriers
+      // result row 4*lg + i of key block kb: key e0 + 16 kb + 4 lg + i
+      if constexpr (FORM == kExtended) {
+        const bool far = bias_h != nullptr && i0 - (e0 + kTileK - 1) >= p.bias_len - 1;      // all of the tile at the last bias
+        const float bias_far = far ? (bias_cached ? bias_lds[wave * p.bias_len + p.bias_len - 1] : bias_h[p.bias_len - 1]) : 0.0f;
+#pragma unroll
+        for (int kb = 0; kb < 4; ++kb) {
+          const f32x4_t ks = *reinterpret_cast<const f32x4_t*>(ks_lds + kb * 16 + 4 * lg);
+          s[kb] = s[kb] * (ks * p.scale) + bias_far;
+        }
+        if (bias_h != nullptr && !far) {
+#pragma unroll
+          for (int kb = 0; kb < 4; ++kb)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+              const int dist = min(max(pos - (e0 + kb * 16 + 4 * lg + i), 0), p.bias_len - 1);
+              s[kb][i] += bias_cached ? bias_lds[wave * p.bias_len + dist] : bias_h[dist];
+            }
+        }
+      } else {
+#pragma unroll
+        for (int kb = 0; kb < 4; ++kb)
+#pragma unroll
+          for (int i = 0; i < 4; ++i) s[kb][i] = FORM == kCapped ? p.cap * fast_tanh(s[kb][i] * p.cap_in) : s[kb][i] * p.scale;
+      }
+      // a tile of tokens that every query of the workgroup sees whole needs no mask
+      const bool whole = phase == 1 && e0 + kTileK - 1 <= i0 && (chunk > 0 ? e0 >= i1 - i1 % chunk : i1 - e0 < W);
+      if (!whole) {
+#pragma unroll
+        for (int kb = 0; kb < 4; ++kb)
+#pragma unroll
+          for (int i = 0; i < 4; ++i) {
+            const int ke = e0 + kb * 16 + 4 * lg + i;
+            bool vis = ke < e_end;
+            if (phase == 0) vis = vis && (P == 0 || ke * P + P - 1 <= pos - W);
+            else vis = vis && ke <= pos && ((chunk > 0 ? ke >= cstart : pos - ke < W) || ke < keep);
+            s[kb][i] = vis ? s[kb][i] : -INFINITY;
+          }
+      }
       float mx = -INFINITY;
 #pragma unroll
       for (int kb = 0; kb < 4; ++kb)
@@ -288,14 +311,14 @@ __global__ __launch_bounds__(256, AHEAD ? 1 : (DVB > 8 ? 2 : (DVB > 4 ? 3 : 4)))
       mx = fmaxf(mx, __shfl_xor(mx, 16, kWave));
       mx = fmaxf(mx, __shfl_xor(mx, 32, kWave));
       const float nm = fmaxf(m, mx);
-      const float corr = expf(m - nm);
+      const float corr = __expf(m - nm);
       float rs = 0.0f;
       bf16x8_t pb[2];                                                       // key blocks (0, 1) and (2, 3) side by side
 #pragma unroll
       for (int kb = 0; kb < 4; ++kb) {
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-          const float e = expf(s[kb][i] - nm);                              // exp(-inf) = 0 for what is not seen
+          const float e = __expf(s[kb][i] - nm);                            // exp(-inf) = 0 for what is not seen
           rs += e;
           pb[kb >> 1][(kb & 1) * 4 + i] = static_cast<__bf16>(e);
         }
