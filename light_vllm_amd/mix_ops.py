@@ -22,6 +22,7 @@ _DT = {torch.bfloat16: 0, torch.float32: 1}
 # windowed pooled attention: "auto" takes the matrix-core kernel where it applies (bf16, head sizes that
 # are multiples of 16 up to 256) and the vector kernel elsewhere (f32, other head sizes); "valu" forces the latter
 WINDOW_ATTN_KERNEL = "auto"
+SPLIT_WORKGROUPS = 256     # decode-shaped attention: key tiles are cut until a launch has about this many workgroups
 
 
 def _stream(t: torch.Tensor) -> int:
@@ -447,7 +448,7 @@ def window_pool_attention(q, k_cache, v_cache, kp, vp, gate, step, H, G, D, Dv, 
                 most = max(c + n for c, n in zip(step.host_ctx_lens, step.host_lens_q))
                 span = min(most, chunk + 16) if chunk > 0 else min(most, window + 16 + keep_first)
                 tiles = -(-span // 64) + (-(-(max(most - window, 0) // P) // 64) if P > 0 else 0)
-                nsplit = max(1, min(tiles, 256 // max(B * G * -(-(H // G) // 4), 1), 32))      # one workgroup a CU: more splits cost more in the merge than they gain (measured)
+                nsplit = max(1, min(tiles, SPLIT_WORKGROUPS // max(B * G * -(-(H // G) // 4), 1), 32))      # one workgroup a CU: more splits cost more in the merge than they gain (measured)
                 if nsplit > 1:
                     ws = torch.empty(T * H * nsplit * (Dv + 4), dtype=torch.float32, device=q.device)
             _mixlib.check(lib.lv_masked_attn_mfma(_p(q), _p(k_cache), _p(v_cache), _p(kp), _p(vp), _p(gate),
